@@ -612,7 +612,9 @@ typedef struct vlm_recurrence_args {
   long ldo;
   int H, D, Dv, gated;
   const void *fbias, *lower;            /* gated = 2: T [H * D] each (fbias may be NULL; lower NULL = 0) */
-  int q_act;                            /* gated = 2: 0 = q as projected, 1 = silu(q) */
+  int q_act;                            /* gated = 0 / 2: 0 = q as projected, 1 = silu(q) */
+  int k_act, v_act;                     /* ABI v13, gated = 0 without rotation: 1 = silu(k) / silu(v) */
+  int row_norm;                         /* ABI v13, gated = 0: ONE RMS norm over all heads of the token instead of one per head */
 } vlm_recurrence_args;
 int vlm_linear_recurrence(const vlm_recurrence_args* a, int nseg, int ntok, int dtype, void* stream);
 
@@ -650,8 +652,9 @@ int vlm_moe_route_scored(const void* logits, int T, int E, int top, int groups, 
  * every token uses).  Outputs as vlm_moe_route. */
 int vlm_moe_route_sigmoid(const void* logits, long ldz, int T, int E, int top, int groups, int keep, int group_top, const void* correction,
                           int normalise, float scale, int extra, void* extra_out, void* gate, void* idx, void* wgt, void* stream);
-int vlm_glu_rows(const void* g, long ldg, const void* u, long ldu, const void* route, int E, int ff, int estride, int act, void* out,
-                 long ldo, int rows, int dim, int dtype, void* stream);
+/* ABI v13: act 3 = clamped gate: g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit). */
+int vlm_glu_rows(const void* g, long ldg, const void* u, long ldu, const void* route, int E, int ff, int estride, int act, float limit,
+                 void* out, long ldo, int rows, int dim, int dtype, void* stream);
 int vlm_moe_relu2_gate(const void* up, long ldu, const void* gate, int E, int ff, int shared, void* out, long ldo, int rows, int dtype,
                        void* stream);
 
@@ -782,6 +785,68 @@ typedef struct vlm_short_conv_args {
 } vlm_short_conv_args;
 int vlm_short_conv_rows(const vlm_short_conv_args* a, int ntok, int dtype, void* stream);
 int vlm_short_conv_carry(const vlm_short_conv_args* a, int nseg, int dtype, void* stream);
+
+/* csrc/short_conv.hip (ABI v13): the same convolution over packed projection rows [q | k | v], then rotary positions on the first
+ * rot_dims dimensions of every head of q and k (pairs (i, i + rot_dims / 2), angle pos * inv_freq[i], cos and sin times amp), q to
+ * dense fp32 rows [HQ * D], k (fp32 [HK * D]) and v (T [NV]) to the token's place in the paged pools.  The carry covers all C columns of
+ * the packed row; vlm_short_conv_carry over the same rows moves it.  taps = 0: no convolution. */
+typedef struct vlm_conv_qkv_args {
+  const void* x;                        /* T rows [C] at ldx */
+  long ldx;
+  const void* w;                        /* T [C][taps] */
+  const float* carry;                   /* fp32 [slots][taps - 1][C] */
+  int C, taps, qoff, koff, voff;        /* first columns of the parts */
+  int HQ, HK, D, NV, rot_dims;
+  const float* inv_freq;
+  float amp;
+  const int *tok_seq, *tok_pos, *block_table;
+  int max_pages;
+  float *q, *kpool;
+  void* vpool;
+} vlm_conv_qkv_args;
+int vlm_conv_qkv_rows(const vlm_conv_qkv_args* a, int ntok, int dtype, void* stream);
+
+/* csrc/diff_attn.hip (ABI v13): attention whose heads are the difference of two softmax maps over the same values, with a sliding
+ * window that keeps the first `keep` tokens in view (window <= 0: causal), RMS norm (no weight) of the difference per head, times mult:
+ *   d = softmax(q1 k1^T scale) v - lambda softmax(q2 k2^T scale) v      out = d / sqrt(mean(d^2) + eps) * mult
+ * _blocks: query blocks of up to 16 consecutive tokens of one sequence (prompt form); _rows: one token per workgroup and head group. */
+typedef struct vlm_diff_attn_args {
+  const float* q;                       /* [tokens][H][2][D] */
+  const float* kpool;                   /* [pages][64][KH][2][D] */
+  const void* vpool;                    /* T [pages][64][KH][Dv] */
+  const int *qb_start, *qb_count;       /* _blocks only */
+  const int *tok_seq, *tok_pos, *block_table;
+  int max_pages, H, KH, D, Dv;
+  float scale;
+  int window, keep;
+  float lambda, mult, eps;
+  void* out;                            /* T rows [H * Dv] at ldo */
+  long ldo;
+} vlm_diff_attn_args;
+int vlm_diff_attn_blocks(const vlm_diff_attn_args* a, int nblocks, int dtype, void* stream);
+int vlm_diff_attn_rows(const vlm_diff_attn_args* a, int rows, int dtype, void* stream);
+
+/* csrc/hyper_stream.hip (ABI v13): S residual streams per token, fp32 [rows][S][D], written and read in one pass:
+ *   x'_t = sum_s mix[s][t] x_s + out[t] y  (y NULL: streams as they are)      h = rms(sum_t in[t] x'_t) * w  (w NULL: no read;
+ * in NULL: every weight one).  xin: stream s of row r at xin + r * xin_tok + s * xin_stream (xin_stream = 0: one row stands for all). */
+typedef struct vlm_hyper_args {
+  const float* xin;
+  long xin_tok, xin_stream;
+  float* xout;                          /* [rows][S][D]; may be xin */
+  const void* y;                        /* T rows [D] at ldy or NULL */
+  long ldy;
+  const float *mix, *out, *in;          /* fp32 [S][S] (from, to), [S], [S] */
+  const void* w;                        /* T [D] or NULL */
+  void* h;                              /* T rows [D] at ldh */
+  long ldh;
+  int S, D;
+  float eps;
+} vlm_hyper_args;
+int vlm_hyper_step(const vlm_hyper_args* a, int rows, int dtype, void* stream);
+
+/* csrc/stream_f32.hip (ABI v13): out = cap * tanh(scale * x / cap), or scale * x with cap = 0; rows fp32 or bf16, in place allowed */
+int vlm_logit_cap_rows(const void* x, long ldx, int x_f32, void* out, long ldo, int out_f32, int rows, int dim, float scale, float cap,
+                       void* stream);
 
 /* csrc/selective_scan.hip (ABI v12): the selective state-space scan, state fp32 [slots][C][N] carried per sequence:
  *   dt = softplus(dt_pre + dt_bias)      S[c][n] <- exp(dt_c A[c][n]) S[c][n] + dt_c x_c B_n      A = -exp(A_log)

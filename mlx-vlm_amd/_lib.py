@@ -100,7 +100,8 @@ class RecurrenceArgs(C.Structure):
                    ("kscale", c_float), ("normw", c_void_p), ("gate_act", c_int), ("eps", c_float), ("seg_start", c_void_p),
                    ("seg_slot", c_void_p), ("seg_pos0", c_void_p), ("state", c_void_p), ("mstate", c_void_p), ("mtok", c_void_p),
                    ("mprev", c_void_p), ("raw", c_void_p), ("out", c_void_p), ("ldo", C.c_long), ("H", c_int), ("D", c_int),
-                   ("Dv", c_int), ("gated", c_int), ("fbias", c_void_p), ("lower", c_void_p), ("q_act", c_int)])
+                   ("Dv", c_int), ("gated", c_int), ("fbias", c_void_p), ("lower", c_void_p), ("q_act", c_int), ("k_act", c_int), ("v_act", c_int),
+                   ("row_norm", c_int)])
 
 
 class DeltaPrepGeneralArgs(C.Structure):
@@ -140,6 +141,28 @@ class ShortConvArgs(C.Structure):
                 ("act", c_int), ("residual", c_int), ("carry", c_void_p), ("tok_seq", c_void_p), ("tok_pos", c_void_p),
                 ("seg_start", c_void_p), ("seg_slot", c_void_p), ("seg_pos0", c_void_p), ("out", c_void_p), ("ldo", C.c_long),
                 ("out_f32", c_int)]
+
+
+class ConvQkvArgs(C.Structure):
+    """vlm_conv_qkv_args (include/vlm_hip.h)"""
+    _fields_ = ([("x", c_void_p), ("ldx", C.c_long), ("w", c_void_p), ("carry", c_void_p)]
+                + [(n, c_int) for n in ("C", "taps", "qoff", "koff", "voff", "HQ", "HK", "D", "NV", "rot_dims")]
+                + [("inv_freq", c_void_p), ("amp", c_float), ("tok_seq", c_void_p), ("tok_pos", c_void_p), ("block_table", c_void_p),
+                   ("max_pages", c_int), ("q", c_void_p), ("kpool", c_void_p), ("vpool", c_void_p)])
+
+
+class DiffAttnArgs(C.Structure):
+    """vlm_diff_attn_args (include/vlm_hip.h)"""
+    _fields_ = ([(n, c_void_p) for n in ("q", "kpool", "vpool", "qb_start", "qb_count", "tok_seq", "tok_pos", "block_table")]
+                + [(n, c_int) for n in ("max_pages", "H", "KH", "D", "Dv")] + [("scale", c_float), ("window", c_int), ("keep", c_int)]
+                + [(n, c_float) for n in ("lam", "mult", "eps")] + [("out", c_void_p), ("ldo", C.c_long)])
+
+
+class HyperArgs(C.Structure):
+    """vlm_hyper_args (include/vlm_hip.h)"""
+    _fields_ = [("xin", c_void_p), ("xin_tok", C.c_long), ("xin_stream", C.c_long), ("xout", c_void_p), ("y", c_void_p), ("ldy", C.c_long),
+                ("mix", c_void_p), ("out", c_void_p), ("in_", c_void_p), ("w", c_void_p), ("h", c_void_p), ("ldh", C.c_long), ("S", c_int),
+                ("D", c_int), ("eps", c_float)]
 
 
 class SelectiveScanArgs(C.Structure):
@@ -249,8 +272,13 @@ SIGNATURES = {
                                        c_void_p, c_int, c_void_p]),
     "vlm_moe_route": (c_int, [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p]),
     "vlm_moe_route_scored": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_void_p]),
-    "vlm_glu_rows": (c_int, [c_void_p, C.c_long, c_void_p, C.c_long, c_void_p, c_int, c_int, c_int, c_int, c_void_p, C.c_long, c_int,
+    "vlm_glu_rows": (c_int, [c_void_p, C.c_long, c_void_p, C.c_long, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p, C.c_long, c_int,
                              c_int, c_int, c_void_p]),
+    "vlm_conv_qkv_rows": (c_int, [P(ConvQkvArgs), c_int, c_int, c_void_p]),
+    "vlm_diff_attn_blocks": (c_int, [P(DiffAttnArgs), c_int, c_int, c_void_p]),
+    "vlm_diff_attn_rows": (c_int, [P(DiffAttnArgs), c_int, c_int, c_void_p]),
+    "vlm_hyper_step": (c_int, [P(HyperArgs), c_int, c_int, c_void_p]),
+    "vlm_logit_cap_rows": (c_int, [c_void_p, C.c_long, c_int, c_void_p, C.c_long, c_int, c_int, c_int, c_float, c_float, c_void_p]),
     "vlm_scaled_add_rms": (c_int, [c_void_p, c_void_p, C.c_long, c_float, c_void_p, C.c_long, c_float, c_void_p, c_float, c_void_p, C.c_long,
                                    c_int, c_int, c_int, c_float, c_int, c_void_p]),
     "vlm_moe_route_sigmoid": (c_int, [c_void_p, C.c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_float, c_int,

@@ -4,6 +4,7 @@
 //
 //   * fixed decay ("retention"): a_t = decay[h], b_t = 1, rotary positions on q and k (rotate-half pairing on the first
 //     rot_dims dimensions), k scaled after the rotation;
+//     or without rotation ("lightning"): silu on q, k and v on the way into LDS (q_act / k_act / v_act);
 //   * gated ("mLSTM"): log input gate i_t = cap * tanh((i~ + bias) / cap), log forget gate f_t = logsigmoid(cap * tanh((f~ +
 //     bias) / cap)), running maximum m_t = max(f_t + m_(t-1), i_t) with m_0 = 0, a_t = exp(f_t + m_(t-1) - m_t),
 //     b_t = exp(i_t - m_t); the normaliser n_t = a_t n_(t-1) + b_t k_t rides along as one more COLUMN of S (v extended by a
@@ -16,7 +17,7 @@
 // sequence; its state is read from the sequence's slot (zero when the segment starts at position 0 - a slot that is used
 // again needs no clearing), advanced token by token with the same arithmetic wherever the prompt was cut, and written back.
 // vlm_linear_recurrence writes the raw o (and n . q) in fp32; vlm_recurrence_finish then applies the denominator, the
-// per-head unit-RMS norm, an optional weight and the output gate (silu or sigmoid of a projection) into a T-typed row.
+// per-head unit-RMS norm (row_norm: ONE norm over all heads of the token), an optional weight and the output gate (silu or sigmoid of a projection) into a T-typed row.
 //
 // Work split: workgroup = (segment, head, tile of 64 state columns); lane c of part p holds rows [32 p, 32 p + 32) of column
 // c in registers.  Tokens are staged 4 / 8 / 16 at a time through LDS (q, k rotated and scaled on the way in).
@@ -89,6 +90,8 @@ __global__ __launch_bounds__(1024) void linear_recurrence_kernel(vlm_recurrence_
           fs[idx] = f;
           kv = 1.f - f;
         } else {
+          if (MODE == 0 && p.q_act == 1) qv = qv / (1.f + expf(-qv));
+          if (MODE == 0 && p.k_act == 1) kv = kv / (1.f + expf(-kv));
           qv *= p.qscale;
           kv *= p.kscale;
         }
@@ -100,7 +103,9 @@ __global__ __launch_bounds__(1024) void linear_recurrence_kernel(vlm_recurrence_
     }
     for (int idx = tid; idx < nb * CT; idx += nthr) {
       const int t = idx / CT, c = c0 + idx % CT;
-      vs[idx] = c < Dv ? ld_f(v + (long)(t0 + t) * p.ldv + c) : (c == Dv && GATED ? 1.f : 0.f);
+      float vv = c < Dv ? ld_f(v + (long)(t0 + t) * p.ldv + c) : (c == Dv && GATED ? 1.f : 0.f);
+      if (MODE == 0 && p.v_act == 1) vv = vv / (1.f + expf(-vv));
+      vs[idx] = vv;
     }
     if (GATED) {
       if (tid < nb) {
@@ -236,7 +241,10 @@ int run(const vlm_recurrence_args& a, int nseg, int ntok, hipStream_t st) {
     hipLaunchKernelGGL((linear_recurrence_kernel<T, 0>), grid, block, lds(TB), st, a, P, TB);
   }
   VLM_CHECK_LAUNCH();
-  if (gated)
+  if (a.row_norm)
+    hipLaunchKernelGGL(recurrence_finish_row_kernel<T>, dim3(ntok), dim3(256), 0, st, a.raw, a.H * a.Dv, a.eps, (const T*)a.g, a.ldg,
+                       (const T*)a.normw, a.gate_act, (T*)a.out, a.ldo);
+  else if (gated)
     hipLaunchKernelGGL((recurrence_finish_kernel<T, true>), dim3(ntok, a.H), dim3(64), 0, st, a.raw, a.H, a.Dv, a.mtok, a.eps,
                        (const T*)a.g, a.ldg, (const T*)a.normw, a.gate_act, (T*)a.out, a.ldo);
   else
@@ -251,6 +259,8 @@ int run(const vlm_recurrence_args& a, int nseg, int ntok, hipStream_t st) {
 extern "C" int vlm_linear_recurrence(const vlm_recurrence_args* a, int nseg, int ntok, int dtype, void* stream) {
   if (!a || nseg < 0 || ntok < 0) return VLM_ERR_ARG;
   if (a->gated < 0 || a->gated > 2 || a->gate_act < 0 || a->gate_act > 2 || (a->gated == 2 && a->rot_dims)) return VLM_ERR_ARG;
+  if (a->gated == 0 && a->rot_dims && (a->q_act || a->k_act)) return VLM_ERR_ARG;       // (no design rotates activated keys)
+  if (a->gated && (a->k_act || a->v_act || a->row_norm)) return VLM_ERR_ARG;
   if (!a->q || !a->k || !a->v || (!a->g && a->gate_act != 2) || !a->state || !a->raw || !a->out || !a->seg_start || !a->seg_slot || !a->seg_pos0)
     return VLM_ERR_ARG;
   if (a->H <= 0 || a->D <= 0 || a->Dv <= 0 || a->rot_dims < 0 || a->rot_dims > a->D || (a->rot_dims & 1)) return VLM_ERR_ARG;

@@ -16,7 +16,8 @@
 //                        scores (not even when the kept ones are negative); weights = the chosen s, divided by their sum + 1e-20
 //                        (when normalise), times scale.  The sigmoid of `extra` further logit columns is handed out beside the
 //                        table: the gate of an expert that every token uses.
-//   vlm_glu_rows         out[t][c] = act(g[t][c]) * u[t][c]; act: 0 = tanh-form gelu, 1 = silu, 2 = sigmoid.  With a route table:
+//   vlm_glu_rows         out[t][c] = act(g[t][c]) * u[t][c]; act: 0 = tanh-form gelu, 1 = silu, 2 = sigmoid, 3 = clamped
+//                        gate: with g' = min(g, limit), u' = clamp(u, -limit, limit): g' sigmoid(1.702 g') (u' + 1).  With a route table:
 //                        E stacked experts of ff output columns, out[t][e ff + j] = act(g[t][e estride + j]) * u[t][e estride + j]
 //                        * route[t][e] (estride: the distance of two experts' columns in g and u, e.g. 2 ff when every expert's
 //                        gate and up rows lie side by side); T-typed in and out, fp32 inside
@@ -248,10 +249,16 @@ __device__ __forceinline__ float glu_act(float z, int act) {
   return act == 1 ? z * sg : sg;
 }
 
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void glu_rows_kernel(const T* __restrict__ g, long ldg, const T* __restrict__ u, long ldu,
                                                        const float* __restrict__ route, int E, int ff, int estride, int act,
-                                                       T* __restrict__ out, long ldo, int rows, int dim) {
+                                                       float limit, T* __restrict__ out, long ldo, int rows, int dim) {
   const long i = (long)blockIdx.x * 256 + threadIdx.x;
   if (i >= (long)rows * dim) return;
   const long t = i / dim;
@@ -267,7 +274,30 @@ __global__ __launch_bounds__(256) void glu_rows_kernel(const T* __restrict__ g, 
     }
     cs = (long)e * estride + (c - e * ff);
   }
-  st_f(out + t * ldo + c, glu_act(ld_f(g + t * ldg + cs), act) * ld_f(u + t * ldu + cs) * r);
+  const float gv = ld_f(g + t * ldg + cs), uv = ld_f(u + t * ldu + cs);
+  st_f(out + t * ldo + c, (act == 3 ? clamped_glu(gv, uv, limit) : glu_act(gv, act) * uv) * r);
+}
+
+// the clamped gate on rows whose columns come in whole groups of 8 (16-byte accesses), no route table
+__device__ __forceinline__ void load8f(const bf16_t* p, float* f) {
+  const uint4 v = *reinterpret_cast<const uint4*>(p);
+  f[0] = bf_lo(v.x); f[1] = bf_hi(v.x); f[2] = bf_lo(v.y); f[3] = bf_hi(v.y);
+  f[4] = bf_lo(v.z); f[5] = bf_hi(v.z); f[6] = bf_lo(v.w); f[7] = bf_hi(v.w);
+}
+__global__ __launch_bounds__(256) void clamped_glu_vec_kernel(const bf16_t* __restrict__ g, long ldg, const bf16_t* __restrict__ u, long ldu,
+                                                              float limit, bf16_t* __restrict__ out, long ldo, int rows, int dim8) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (long)rows * dim8) return;
+  const long t = i / dim8;
+  const int c = (int)(i % dim8) * 8;
+  float gv[8], uv[8];
+  load8f(g + t * ldg + c, gv);
+  load8f(u + t * ldu + c, uv);
+  unsigned o[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    o[j] = pack_bf2(clamped_glu(gv[2 * j], uv[2 * j], limit), clamped_glu(gv[2 * j + 1], uv[2 * j + 1], limit));
+  *reinterpret_cast<uint4*>(out + t * ldo + c) = make_uint4(o[0], o[1], o[2], o[3]);
 }
 
 }  // namespace
@@ -311,8 +341,8 @@ extern "C" int vlm_moe_route_sigmoid(const void* logits, long ldz, int T, int E,
 }
 
 extern "C" int vlm_glu_rows(const void* g, long ldg, const void* u, long ldu, const void* route, int E, int ff, int estride, int act,
-                            void* out, long ldo, int rows, int dim, int dtype, void* stream) {
-  if (!g || !u || !out || rows < 0 || dim <= 0 || ldo < dim || act < 0 || act > 2) return VLM_ERR_ARG;
+                            float limit, void* out, long ldo, int rows, int dim, int dtype, void* stream) {
+  if (!g || !u || !out || rows < 0 || dim <= 0 || ldo < dim || act < 0 || act > 3 || (act == 3 && !(limit >= 0.f))) return VLM_ERR_ARG;
   if (route ? (E <= 0 || ff <= 0 || (long)E * ff != dim || estride < ff || ldg < (long)(E - 1) * estride + ff ||
                ldu < (long)(E - 1) * estride + ff)
             : (ldg < dim || ldu < dim))
@@ -320,12 +350,20 @@ extern "C" int vlm_glu_rows(const void* g, long ldg, const void* u, long ldu, co
   if (rows == 0) return VLM_OK;
   const unsigned nb = (unsigned)(((long)rows * dim + 255) / 256);
   hipStream_t st = (hipStream_t)stream;
+  if (act == 3 && !dtype && !route && dim % 8 == 0 && ldg % 8 == 0 && ldu % 8 == 0 && ldo % 8 == 0 &&
+      (((uintptr_t)g | (uintptr_t)u | (uintptr_t)out) & 15) == 0) {
+    const unsigned nv = (unsigned)(((long)rows * (dim / 8) + 255) / 256);
+    hipLaunchKernelGGL(clamped_glu_vec_kernel, dim3(nv), dim3(256), 0, st, (const bf16_t*)g, ldg, (const bf16_t*)u, ldu, limit, (bf16_t*)out,
+                       ldo, rows, dim / 8);
+    VLM_CHECK_LAUNCH();
+    return VLM_OK;
+  }
   if (dtype)
     hipLaunchKernelGGL(glu_rows_kernel<float>, dim3(nb), dim3(256), 0, st, (const float*)g, ldg, (const float*)u, ldu, (const float*)route,
-                       E, ff, estride, act, (float*)out, ldo, rows, dim);
+                       E, ff, estride, act, limit, (float*)out, ldo, rows, dim);
   else
     hipLaunchKernelGGL(glu_rows_kernel<bf16_t>, dim3(nb), dim3(256), 0, st, (const bf16_t*)g, ldg, (const bf16_t*)u, ldu,
-                       (const float*)route, E, ff, estride, act, (bf16_t*)out, ldo, rows, dim);
+                       (const float*)route, E, ff, estride, act, limit, (bf16_t*)out, ldo, rows, dim);
   VLM_CHECK_LAUNCH();
   return VLM_OK;
 }

@@ -48,4 +48,31 @@ __global__ __launch_bounds__(64) void recurrence_finish_kernel(const float* __re
   }
 }
 
+// the same with ONE norm over all heads of a token (N = heads * Dv values): grid (tokens), 256 lanes
+template <typename T>
+__global__ __launch_bounds__(256) void recurrence_finish_row_kernel(const float* __restrict__ raw, int N, float eps, const T* __restrict__ g,
+                                                                    long ldg, const T* __restrict__ normw, int gate_act,
+                                                                    T* __restrict__ out, long ldo) {
+  __shared__ float red[4];
+  const long tok = blockIdx.x;
+  const float* o = raw + tok * N;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < N; c += 256) ss += o[c] * o[c];
+  ss = wave_sum(ss);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+  __syncthreads();
+  const float r = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)N + eps);
+  const T* gp = g + tok * ldg;
+  T* op = out + tok * ldo;
+  for (int c = threadIdx.x; c < N; c += 256) {
+    float x = o[c] * r;
+    if (normw) x *= ld_f(normw + c);
+    if (gate_act != 2) {
+      const float gv = ld_f(gp + c), sg = 1.f / (1.f + expf(-gv));
+      x *= gate_act == 0 ? gv * sg : sg;
+    }
+    st_f(op + c, x);
+  }
+}
+
 }  // namespace

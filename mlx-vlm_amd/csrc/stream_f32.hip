@@ -19,6 +19,8 @@
 //                              x[t] += mult * y[t] (+ mult2 * y2[t])                  (y may be NULL: norm only)
 //                              h[t] = x[t] * rsqrt(mean(x[t]^2) + eps) * (w_offset + w)   (w may be NULL: add only; w_offset 1
 //                                                                                      for weights kept as offsets from one)
+//   vlm_logit_cap_rows       out[t][j] = cap * tanh(scale * x[t][j] / cap)    (cap = 0: scale * x alone); x and out each fp32 or bf16, may be
+//                                                                                      the same rows
 #include "common.hpp"
 #include "../../include/vlm_hip.h"
 
@@ -199,6 +201,16 @@ __global__ __launch_bounds__(256) void relu2_rows_kernel(const T* __restrict__ i
   st_f(out + t * ldo + j, v * v);
 }
 
+template <typename TI, typename TO>
+__global__ __launch_bounds__(256) void logit_cap_kernel(const TI* x, long ldx, TO* out, long ldo, int dim, float scale,
+                                                        float cap) {
+  const int j = blockIdx.x * 256 + threadIdx.x;
+  if (j >= dim) return;
+  float v = ld_f(x + (long)blockIdx.y * ldx + j) * scale;
+  if (cap > 0.f) v = cap * tanhf(v / cap);
+  st_f(out + (long)blockIdx.y * ldo + j, v);
+}
+
 }  // namespace
 
 #define STREAM_ARGS_OK(rows, D) ((rows) >= 0 && (D) > 0)
@@ -319,6 +331,24 @@ extern "C" int vlm_scaled_add_rms(void* x, const void* y, long ldy, float mult, 
   if (dtype) hipLaunchKernelGGL((scaled_add_rms_kernel<float, float>), dim3(rows), dim3(256), 0, st, (float*)x, (const float*)y, ldy, mult, (const float*)y2, ldy2, mult2, (const float*)w, w_offset, (float*)h, ldh, D, eps);
   else if (h_f32) hipLaunchKernelGGL((scaled_add_rms_kernel<bf16_t, float>), dim3(rows), dim3(256), 0, st, (float*)x, (const bf16_t*)y, ldy, mult, (const bf16_t*)y2, ldy2, mult2, (const bf16_t*)w, w_offset, (float*)h, ldh, D, eps);
   else hipLaunchKernelGGL((scaled_add_rms_kernel<bf16_t, bf16_t>), dim3(rows), dim3(256), 0, st, (float*)x, (const bf16_t*)y, ldy, mult, (const bf16_t*)y2, ldy2, mult2, (const bf16_t*)w, w_offset, (bf16_t*)h, ldh, D, eps);
+  VLM_CHECK_LAUNCH();
+  return VLM_OK;
+}
+
+extern "C" int vlm_logit_cap_rows(const void* x, long ldx, int x_f32, void* out, long ldo, int out_f32, int rows, int dim, float scale, float cap,
+                                  void* stream) {
+  if (!x || !out || rows < 0 || dim <= 0 || ldx < dim || ldo < dim || !(cap >= 0.f) || (x == out && (!x_f32 != !out_f32 || ldx != ldo))) return VLM_ERR_ARG;
+  if (rows > 65535) return VLM_ERR_SHAPE;
+  if (rows == 0) return VLM_OK;
+  hipStream_t st = (hipStream_t)stream;
+  dim3 grid((dim + 255) / 256, rows);
+#define GO(TI, TO) hipLaunchKernelGGL((logit_cap_kernel<TI, TO>), grid, dim3(256), 0, st, (const TI*)x, ldx, (TO*)out, ldo, dim, scale, cap)
+  if (x_f32) {
+    if (out_f32) GO(float, float); else GO(float, bf16_t);
+  } else {
+    if (out_f32) GO(bf16_t, float); else GO(bf16_t, bf16_t);
+  }
+#undef GO
   VLM_CHECK_LAUNCH();
   return VLM_OK;
 }

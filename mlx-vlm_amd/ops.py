@@ -711,18 +711,18 @@ def moe_route_scored(logits, top, groups=1, keep=1, scale=1.0):
     return gate, idx, wgt
 
 
-GLU_GELU_TANH, GLU_SILU, GLU_SIGMOID = 0, 1, 2
+GLU_GELU_TANH, GLU_SILU, GLU_SIGMOID, GLU_CLAMPED = 0, 1, 2, 3
 
 
-def glu_rows(g, u, act, out=None, route=None, E=0, ff=0, estride=0):
-    """out = act(g) * u over 2-D views with a row pitch (dim: out's columns, else g's); with route (fp32 [T, E]): out [T, E * ff], expert e reads the
+def glu_rows(g, u, act, out=None, route=None, E=0, ff=0, estride=0, limit=float("inf")):
+    """out = act(g) * u (GLU_CLAMPED: g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' within +-limit) over 2-D views with a row pitch (dim: out's columns, else g's); with route (fp32 [T, E]): out [T, E * ff], expert e reads the
     columns e * estride .. + ff of g and u, times route[t, e]"""
     _dev(g, u, out, route)
     rows = g.shape[0]
     dim = int(E) * int(ff) if route is not None else (out.shape[1] if out is not None else g.shape[1])
     if out is None:
         out = torch.empty(rows, dim, dtype=g.dtype, device=g.device)
-    check(_lib.lib().vlm_glu_rows(_p(g), g.stride(0), _p(u), u.stride(0), _p(route), int(E), int(ff), int(estride or ff), int(act),
+    check(_lib.lib().vlm_glu_rows(_p(g), g.stride(0), _p(u), u.stride(0), _p(route), int(E), int(ff), int(estride or ff), int(act), float(limit),
                                   _p(out), out.stride(0), rows, dim, _f32(g), _stream()), "glu_rows")
     return out
 
@@ -921,3 +921,110 @@ def short_conv_rows(x, w, carry, tok_seq, tok_pos, cu, slot, pos0, bias=None, ac
 
 def selective_scan(args: "_lib.SelectiveScanArgs", nseg: int, ntok: int, dtype_f32: bool):
     check(_lib.lib().vlm_selective_scan(C.byref(args), int(nseg), int(ntok), int(bool(dtype_f32)), _stream()), "selective_scan")
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# Hyper-connected residual streams, convolved and rotated q / k / v rows, differential attention, capped logits.
+def hyper_step(xin, S, y=None, mix=None, out=None, w_in=None, w=None, eps=1e-6, xout=None, h=None):
+    """S residual streams per token.  xin: fp32 [T, S, D], or [T, D] when one row stands for all S streams.  With y [T, D]: the new
+    streams sum_s mix[s, t] x_s + out[t] y go to xout ([T, S, D]; default: xin updated in place).  With w: returns
+    h = rms(sum_t w_in[t] x_t) * w in w's dtype (w_in None: the plain sum), else None.  mix / out / w_in: fp32 device tensors."""
+    _dev(xin, y, mix, out, w_in, w, xout, h)
+    if xin.dtype != torch.float32 or not xin.is_contiguous() or (xin.dim() == 3 and xin.shape[1] != S):
+        raise _lib.VlmHipError("hyper_step: contiguous fp32 streams [T, S, D] (or [T, D]) expected")
+    T, D = xin.shape[0], xin.shape[-1]
+    for c, shape in ((mix, (S, S)), (out, (S,)), (w_in, (S,))):
+        if c is not None and (c.dtype != torch.float32 or tuple(c.shape) != shape or not c.is_contiguous()):
+            raise _lib.VlmHipError("hyper_step: fp32 stream weights of S (x S) entries expected")
+    if y is not None:
+        if y.shape != (T, D) or mix is None or out is None:
+            raise _lib.VlmHipError("hyper_step: y [T, D] comes with mix and out")
+        if xout is None:
+            if xin.dim() != 3:
+                raise _lib.VlmHipError("hyper_step: xout is needed when one row stands for all streams")
+            xout = xin
+        if xout.dtype != torch.float32 or tuple(xout.shape) != (T, S, D) or not xout.is_contiguous():
+            raise _lib.VlmHipError("hyper_step: xout is contiguous fp32 [T, S, D]")
+    if w is not None:
+        if w.shape != (D,) or (y is not None and y.dtype != w.dtype):
+            raise _lib.VlmHipError("hyper_step: the norm weight has D entries of y's dtype")
+        if h is None:
+            h = torch.empty(T, D, dtype=w.dtype, device=xin.device)
+    a = _lib.HyperArgs()
+    a.xin, a.xin_tok, a.xin_stream = _p(xin), xin.stride(0), xin.stride(1) if xin.dim() == 3 else 0
+    a.S, a.D, a.eps = int(S), int(D), float(eps)
+    if y is not None:
+        a.xout, a.y, a.ldy, a.mix, a.out = _p(xout), _p(y), y.stride(0), _p(mix), _p(out)
+    if w is not None:
+        a.in_, a.w, a.h, a.ldh = _p(w_in), _p(w), _p(h), h.stride(0)
+    check(_lib.lib().vlm_hyper_step(C.byref(a), T, _f32(y if y is not None else w), _stream()), "hyper_step")
+    return h if w is not None else None
+
+
+def conv_qkv_rows(x, w, carry, offs, HQ, HK, D, NV, tok_seq, tok_pos, cu, slot, pos0, block_table, q, kpool, vpool, rot_dims=0,
+                  inv_freq=None, amp=1.0):
+    """Packed projection rows x [T, C] = [q | k | v] at columns offs -> short causal convolution (w [C, taps], None: none; carry
+    fp32 [slots, taps - 1, C], moved to the end of the step's segments) -> rotate-half positions on the first rot_dims dimensions of the
+    HQ + HK heads of q and k (cos and sin times amp) -> q fp32 [T, HQ * D] and the paged pools (keys fp32, values in x's dtype)."""
+    _dev(x, w, carry, tok_seq, tok_pos, cu, slot, pos0, block_table, q, kpool, vpool, inv_freq)
+    T, C_ = x.shape
+    taps = w.shape[1] if w is not None else 0
+    if (w is not None and (w.shape[0] != C_ or w.dtype != x.dtype or not w.is_contiguous())) or vpool.dtype != x.dtype:
+        raise _lib.VlmHipError("conv_qkv_rows: one filter per packed column and a value pool, both of the rows' dtype, expected")
+    if taps > 1 and (carry is None or carry.dtype != torch.float32 or tuple(carry.shape[1:]) != (taps - 1, C_)):
+        raise _lib.VlmHipError("conv_qkv_rows: fp32 carry [slots, taps - 1, columns] expected")
+    if q.dtype != torch.float32 or kpool.dtype != torch.float32 or q.numel() != T * HQ * D or kpool.shape[-1] != HK * D or vpool.shape[-1] != NV:
+        raise _lib.VlmHipError("conv_qkv_rows: fp32 q rows [T, HQ * D], key pool [.., HK * D], value pool [.., NV] expected")
+    a = _lib.ConvQkvArgs()
+    a.x, a.ldx, a.w, a.carry, a.C, a.taps = _p(x), x.stride(0), _p(w), _p(carry), int(C_), int(taps)
+    a.qoff, a.koff, a.voff = (int(o) for o in offs)
+    a.HQ, a.HK, a.D, a.NV, a.rot_dims, a.inv_freq, a.amp = int(HQ), int(HK), int(D), int(NV), int(rot_dims), _p(inv_freq), float(amp)
+    a.tok_seq, a.tok_pos, a.block_table, a.max_pages = _p(tok_seq), _p(tok_pos), _p(block_table), block_table.shape[1]
+    a.q, a.kpool, a.vpool = _p(q), _p(kpool), _p(vpool)
+    check(_lib.lib().vlm_conv_qkv_rows(C.byref(a), T, _f32(x), _stream()), "conv_qkv_rows")
+    if taps > 1:
+        b = _lib.ShortConvArgs()
+        b.in_, b.ldin, b.in_f32, b.w, b.C, b.taps, b.carry = _p(x), x.stride(0), int(x.dtype == torch.float32), _p(w), int(C_), int(taps), _p(carry)
+        b.seg_start, b.seg_slot, b.seg_pos0 = _p(cu), _p(slot), _p(pos0)
+        check(_lib.lib().vlm_short_conv_carry(C.byref(b), slot.numel(), _f32(x), _stream()), "short_conv_carry")
+    return q
+
+
+def _diff_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window, keep):
+    if q.dtype != torch.float32 or kpool.dtype != torch.float32 or vpool.dtype != out.dtype or not q.is_contiguous():
+        raise _lib.VlmHipError("diff_attn: fp32 queries and keys, values and output of one dtype expected")
+    if kpool.shape[-1] != KH * 2 * D or vpool.shape[-1] != KH * Dv or q.numel() != tok_seq.numel() * H * 2 * D:
+        raise _lib.VlmHipError("diff_attn: two maps of D per head in q and the key pool, Dv value columns per head")
+    a = _lib.DiffAttnArgs()
+    a.q, a.kpool, a.vpool, a.tok_seq, a.tok_pos, a.block_table = _p(q), _p(kpool), _p(vpool), _p(tok_seq), _p(tok_pos), _p(block_table)
+    a.max_pages, a.H, a.KH, a.D, a.Dv, a.scale = block_table.shape[1], int(H), int(KH), int(D), int(Dv), float(scale)
+    a.window, a.keep, a.lam, a.mult, a.eps, a.out, a.ldo = int(window), int(keep), float(lam), float(mult), float(eps), _p(out), out.stride(0)
+    return a
+
+
+def diff_attn_blocks(q, kpool, vpool, qb_start, qb_count, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window=0,
+                     keep=0):
+    """differential attention, prompt form: q fp32 [T, H * 2 * D], pools with rows [KH * 2 * D] / [KH * Dv], out [T, H * Dv];
+    window > 0: a query reaches back window - 1 tokens and to the first `keep` tokens of its sequence"""
+    _dev(q, kpool, vpool, qb_start, qb_count, tok_seq, tok_pos, block_table, out)
+    a = _diff_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window, keep)
+    a.qb_start, a.qb_count = _p(qb_start), _p(qb_count)
+    check(_lib.lib().vlm_diff_attn_blocks(C.byref(a), qb_start.numel(), _f32(vpool), _stream()), "diff_attn_blocks")
+    return out
+
+
+def diff_attn_rows(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window=0, keep=0):
+    """differential attention, decode form (one workgroup per token and group of heads that share a key / value head)"""
+    _dev(q, kpool, vpool, tok_seq, tok_pos, block_table, out)
+    a = _diff_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window, keep)
+    check(_lib.lib().vlm_diff_attn_rows(C.byref(a), tok_seq.numel(), _f32(vpool), _stream()), "diff_attn_rows")
+    return out
+
+
+def logit_cap_rows(x, scale=1.0, cap=0.0, out=None):
+    """cap * tanh(scale * x / cap) (cap 0: scale * x) over 2-D rows, fp32 or bf16; out None: in place"""
+    _dev(x, out)
+    o = x if out is None else out
+    check(_lib.lib().vlm_logit_cap_rows(_p(x), x.stride(0), _f32(x), _p(o), o.stride(0), _f32(o), x.shape[0], x.shape[1], float(scale),
+                                        float(cap), _stream()), "logit_cap_rows")
+    return o
