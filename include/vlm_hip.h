@@ -615,6 +615,8 @@ typedef struct vlm_recurrence_args {
   int q_act;                            /* gated = 0 / 2: 0 = q as projected, 1 = silu(q) */
   int k_act, v_act;                     /* ABI v13, gated = 0 without rotation: 1 = silu(k) / silu(v) */
   int row_norm;                         /* ABI v13, gated = 0: ONE RMS norm over all heads of the token instead of one per head */
+  float* ws;                            /* ABI v13: workspace of the chunk-parallel form (fixed decay without rotation), or NULL */
+  long ws_floats;                       /* its size; H * D * Dv per chunk of 64 tokens (at least one), fewer chunks run in windows */
 } vlm_recurrence_args;
 int vlm_linear_recurrence(const vlm_recurrence_args* a, int nseg, int ntok, int dtype, void* stream);
 

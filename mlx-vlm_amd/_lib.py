@@ -101,7 +101,7 @@ class RecurrenceArgs(C.Structure):
                    ("seg_slot", c_void_p), ("seg_pos0", c_void_p), ("state", c_void_p), ("mstate", c_void_p), ("mtok", c_void_p),
                    ("mprev", c_void_p), ("raw", c_void_p), ("out", c_void_p), ("ldo", C.c_long), ("H", c_int), ("D", c_int),
                    ("Dv", c_int), ("gated", c_int), ("fbias", c_void_p), ("lower", c_void_p), ("q_act", c_int), ("k_act", c_int), ("v_act", c_int),
-                   ("row_norm", c_int)])
+                   ("row_norm", c_int), ("ws", c_void_p), ("ws_floats", C.c_long)])
 
 
 class DeltaPrepGeneralArgs(C.Structure):

@@ -19,11 +19,15 @@
 // vlm_linear_recurrence writes the raw o (and n . q) in fp32; vlm_recurrence_finish then applies the denominator, the
 // per-head unit-RMS norm (row_norm: ONE norm over all heads of the token), an optional weight and the output gate (silu or sigmoid of a projection) into a T-typed row.
 //
+// With a workspace (ws) and no rotation, fixed-decay segments of VLM_CHUNK_MIN tokens or more run chunk-parallel on the matrix
+// cores instead (chunk_recurrence.hip).
+//
 // Work split: workgroup = (segment, head, tile of 64 state columns); lane c of part p holds rows [32 p, 32 p + 32) of column
 // c in registers.  Tokens are staged 4 / 8 / 16 at a time through LDS (q, k rotated and scaled on the way in).
 #include "common.hpp"
 #include "../../include/vlm_hip.h"
 #include "recurrence_finish.hpp"
+#include "chunk_recurrence.hpp"
 
 namespace {
 
@@ -33,7 +37,7 @@ constexpr int CT = 64;       // state columns per workgroup
 __device__ __forceinline__ float logsigmoid_f(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
 
 template <typename T, int MODE>
-__global__ __launch_bounds__(1024) void linear_recurrence_kernel(vlm_recurrence_args p, int P, int TB) {
+__global__ __launch_bounds__(1024) void linear_recurrence_kernel(vlm_recurrence_args p, int P, int TB, int max_len) {
   constexpr bool GATED = MODE == 1, ROWGATE = MODE == 2;
   extern __shared__ __align__(16) float smem[];
   const int seg = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * CT;
@@ -47,6 +51,7 @@ __global__ __launch_bounds__(1024) void linear_recurrence_kernel(vlm_recurrence_
   float* po = ab + TB * 4;                // [TB][P][CT]
   float* fs = po + TB * P * CT;           // [TB][DP] (ROWGATE): the forget gate per state row; ks holds 1 - f
   const int t_begin = p.seg_start[seg], t_end = p.seg_start[seg + 1];
+  if (t_end - t_begin > max_len) return;                 // (the whole workgroup: this segment runs in the chunk-parallel form)
   const int slot = p.seg_slot[seg], pos0 = p.seg_pos0[seg];
   const T* q = (const T*)p.q + (long)h * D;
   const T* k = (const T*)p.k + (long)h * D;
@@ -230,17 +235,26 @@ int run(const vlm_recurrence_args& a, int nseg, int ntok, hipStream_t st) {
   while (TB > 4 && lds(TB) > 48 * 1024) TB >>= 1;
   if (lds(TB) > 64 * 1024) return VLM_ERR_SHAPE;
   dim3 grid(nseg, a.H, (C + CT - 1) / CT), block(P * CT);
+  int max_len = 0x7fffffff;
+  const int longest = ntok - nseg + 1;                   // no segment of the step is longer (every segment has a token)
+  if (!gated && !rowgate && !a.rot_dims && a.ws && longest >= VLM_CHUNK_MIN) {
+    max_len = VLM_CHUNK_MIN - 1;
+    const int rc = vlm_chunk_recurrence(&a, nseg, ntok, max_len, sizeof(T) == 4, st);
+    if (rc) return rc;
+    if (nseg == 1) goto finish;                          // (the one segment is a long one)
+  }
   if (gated) {
     // the per-token maxima first: the scan kernel overwrites the slot's running maximum
     hipLaunchKernelGGL(gate_max_kernel<T>, dim3(nseg * a.H), dim3(64), 0, st, a, nseg);
     VLM_CHECK_LAUNCH();
-    hipLaunchKernelGGL((linear_recurrence_kernel<T, 1>), grid, block, lds(TB), st, a, P, TB);
+    hipLaunchKernelGGL((linear_recurrence_kernel<T, 1>), grid, block, lds(TB), st, a, P, TB, max_len);
   } else if (rowgate) {
-    hipLaunchKernelGGL((linear_recurrence_kernel<T, 2>), grid, block, lds(TB), st, a, P, TB);
+    hipLaunchKernelGGL((linear_recurrence_kernel<T, 2>), grid, block, lds(TB), st, a, P, TB, max_len);
   } else {
-    hipLaunchKernelGGL((linear_recurrence_kernel<T, 0>), grid, block, lds(TB), st, a, P, TB);
+    hipLaunchKernelGGL((linear_recurrence_kernel<T, 0>), grid, block, lds(TB), st, a, P, TB, max_len);
   }
   VLM_CHECK_LAUNCH();
+finish:
   if (a.row_norm)
     hipLaunchKernelGGL(recurrence_finish_row_kernel<T>, dim3(ntok), dim3(256), 0, st, a.raw, a.H * a.Dv, a.eps, (const T*)a.g, a.ldg,
                        (const T*)a.normw, a.gate_act, (T*)a.out, a.ldo);
@@ -263,6 +277,7 @@ extern "C" int vlm_linear_recurrence(const vlm_recurrence_args* a, int nseg, int
   if (a->gated && (a->k_act || a->v_act || a->row_norm)) return VLM_ERR_ARG;
   if (!a->q || !a->k || !a->v || (!a->g && a->gate_act != 2) || !a->state || !a->raw || !a->out || !a->seg_start || !a->seg_slot || !a->seg_pos0)
     return VLM_ERR_ARG;
+  if (a->ws && a->ws_floats < (long)a->H * a->D * a->Dv) return VLM_ERR_ARG;
   if (a->H <= 0 || a->D <= 0 || a->Dv <= 0 || a->rot_dims < 0 || a->rot_dims > a->D || (a->rot_dims & 1)) return VLM_ERR_ARG;
   if (a->rot_dims && !a->inv_freq) return VLM_ERR_ARG;
   if (a->gated == 2 ? false : a->gated ? (!a->ipre || !a->fpre || !a->ib || !a->fb || !a->mstate || !a->mtok || !a->mprev || !(a->cap > 0.f)) : !a->decay) return VLM_ERR_ARG;

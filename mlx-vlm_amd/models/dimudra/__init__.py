@@ -13,5 +13,5 @@ from .dimudra import Model
 __all__ = ["Model", "ModelConfig", "LayerConfig", "LanguageModel"]
 
 # the operator sources (csrc/<name>.hip) the model's step function needs: what a trace replay of a fresh checkout compiles
-HIP_SOURCES = ('gemm_bf16', 'gemm256_bf16', 'linear_any', 'stream_f32', 'moe', 'window_attn', 'linear_recurrence', 'short_conv',
+HIP_SOURCES = ('gemm_bf16', 'gemm256_bf16', 'linear_any', 'stream_f32', 'moe', 'window_attn', 'linear_recurrence', 'chunk_recurrence', 'short_conv',
                'selective_scan')

@@ -12,4 +12,5 @@ from .zivitar import Model
 __all__ = ["Model", "ModelConfig", "LayerConfig", "LanguageModel"]
 
 # the operator sources (csrc/<name>.hip) the model's step function needs: what a trace replay of a fresh checkout compiles
-HIP_SOURCES = ('gemm_bf16', 'gemm256_bf16', 'linear_any', 'stream_f32', 'hyper_stream', 'moe', 'short_conv', 'diff_attn', 'linear_recurrence')
+HIP_SOURCES = ('gemm_bf16', 'gemm256_bf16', 'linear_any', 'stream_f32', 'hyper_stream', 'moe', 'short_conv', 'diff_attn', 'linear_recurrence',
+               'chunk_recurrence')

@@ -143,9 +143,20 @@ class LanguageModel(RaggedLanguageModel):
         a.seg_start, a.seg_slot, a.seg_pos0 = pl.cu.data_ptr(), pl.slot.data_ptr(), pl.pos0.data_ptr()
         a.state, a.raw, a.out, a.ldo = self.pool.state[i].data_ptr(), raw.data_ptr(), out.data_ptr(), out.stride(0)
         a.H, a.D, a.Dv = H, D, Dv
+        ws = self._workspace(pl, H * D * Dv)
+        if ws is not None:
+            a.ws, a.ws_floats = ws.data_ptr(), ws.numel()
         ops.linear_recurrence(a, pl.nseg, Tn, self.dtype == torch.float32)
-        keep.append(raw)
+        keep += [raw, ws]
         return out
+
+    def _workspace(self, pl, entries):
+        """room for the chunk-parallel recurrence of a step with prompt portions: `entries` fp32 values per chunk, up to 256 MB (longer
+        prompts run in windows of chunks)"""
+        if pl.Tn - pl.nseg < 16:                              # decode rows and short portions only
+            return None
+        chunks = pl.Tn // 64 + pl.nseg
+        return torch.empty(min(chunks, max(1, (64 << 20) // entries)) * entries, dtype=torch.float32, device=self.device)
 
     # ------------------------------------------------------------------ the device side of a step
     def _run(self, pl, logits_dtype=torch.float32):

@@ -208,7 +208,9 @@ def test_differential_attention_against_dense_maps(dtype, D, Dv, Hh, G):
 
 @pytest.mark.parametrize("Hh,D,Dv", [(3, 10, 14), (1, 72, 136), (2, 33, 5), (7, 1, 1), (2, 128, 128), (2, 64, 32), (3, 64, 64), (1, 160, 48)])
 @pytest.mark.parametrize("T", [torch.float32, torch.bfloat16])
-def test_fixed_decay_recurrence_in_portions_and_reused_slots(T, Hh, D, Dv):
+@pytest.mark.parametrize("room", [0, 1, 3, 100])
+def test_fixed_decay_recurrence_in_portions_and_reused_slots(T, Hh, D, Dv, room):
+    """room: chunks the workspace of the chunk-parallel form holds (0: token by token; fewer than the step has: windows of chunks)"""
     from mlx_vlm_amd import _lib, ops
 
     g = torch.Generator().manual_seed(D + Dv)
@@ -236,6 +238,9 @@ def test_fixed_decay_recurrence_in_portions_and_reused_slots(T, Hh, D, Dv):
         a.seg_start, a.seg_slot, a.seg_pos0 = cu.data_ptr(), sl.data_ptr(), p0.data_ptr()
         a.state, a.raw, a.out, a.ldo = state.data_ptr(), raw.data_ptr(), out.data_ptr(), out.stride(0)
         a.H, a.D, a.Dv = Hh, D, Dv
+        ws = torch.full((max(room, 1) * Hh * D * Dv,), float("nan"), device="cuda")
+        if room:
+            a.ws, a.ws_floats = ws.data_ptr(), ws.numel()
         ops.linear_recurrence(a, len(parts), ntok, T == torch.float32)
         torch.cuda.synchronize()
         return out.float().cpu()
