@@ -790,7 +790,8 @@ int vlm_short_conv_carry(const vlm_short_conv_args* a, int nseg, int dtype, void
 
 /* csrc/short_conv.hip (ABI v13): the same convolution over packed projection rows [q | k | v], then rotary positions on the first
  * rot_dims dimensions of every head of q and k (pairs (i, i + rot_dims / 2), angle pos * inv_freq[i], cos and sin times amp), q to
- * dense fp32 rows [HQ * D], k (fp32 [HK * D]) and v (T [NV]) to the token's place in the paged pools.  The carry covers all C columns of
+ * dense fp32 rows [HQ * D], k (fp32 [HK * D]; with k_split as bf16 pairs hi + lo, [HK][2][D8], D8 = D rounded up to 8) and v (T [NV]) to
+ * the token's place in the paged pools.  The carry covers all C columns of
  * the packed row; vlm_short_conv_carry over the same rows moves it.  taps = 0: no convolution. */
 typedef struct vlm_conv_qkv_args {
   const void* x;                        /* T rows [C] at ldx */
@@ -803,8 +804,9 @@ typedef struct vlm_conv_qkv_args {
   float amp;
   const int *tok_seq, *tok_pos, *block_table;
   int max_pages;
-  float *q, *kpool;
-  void* vpool;
+  float* q;
+  void *kpool, *vpool;
+  int k_split;
 } vlm_conv_qkv_args;
 int vlm_conv_qkv_rows(const vlm_conv_qkv_args* a, int ntok, int dtype, void* stream);
 
@@ -814,7 +816,8 @@ int vlm_conv_qkv_rows(const vlm_conv_qkv_args* a, int ntok, int dtype, void* str
  * _blocks: query blocks of up to 16 consecutive tokens of one sequence (prompt form); _rows: one token per workgroup and head group. */
 typedef struct vlm_diff_attn_args {
   const float* q;                       /* [tokens][H][2][D] */
-  const float* kpool;                   /* [pages][64][KH][2][D] */
+  const void* kpool;                    /* dtype fp32: fp32 [pages][64][KH][2][D]; bf16: every coordinate as a sum of two bf16 values,
+                                           [pages][64][KH][2][2 (hi, lo)][D8], D8 = D rounded up to 8, padding zero */
   const void* vpool;                    /* T [pages][64][KH][Dv] */
   const int *qb_start, *qb_count;       /* _blocks only */
   const int *tok_seq, *tok_pos, *block_table;
@@ -824,6 +827,8 @@ typedef struct vlm_diff_attn_args {
   float lambda, mult, eps;
   void* out;                            /* T rows [H * Dv] at ldo */
   long ldo;
+  int nsplit;                           /* _rows: workgroups that share a column group's keys (0 / 1: one; at most 64) */
+  float* part;                          /* nsplit > 1: scratch fp32 [nsplit][H][rows][2][Dv + 2] */
 } vlm_diff_attn_args;
 int vlm_diff_attn_blocks(const vlm_diff_attn_args* a, int nblocks, int dtype, void* stream);
 int vlm_diff_attn_rows(const vlm_diff_attn_args* a, int rows, int dtype, void* stream);

@@ -148,14 +148,14 @@ class ConvQkvArgs(C.Structure):
     _fields_ = ([("x", c_void_p), ("ldx", C.c_long), ("w", c_void_p), ("carry", c_void_p)]
                 + [(n, c_int) for n in ("C", "taps", "qoff", "koff", "voff", "HQ", "HK", "D", "NV", "rot_dims")]
                 + [("inv_freq", c_void_p), ("amp", c_float), ("tok_seq", c_void_p), ("tok_pos", c_void_p), ("block_table", c_void_p),
-                   ("max_pages", c_int), ("q", c_void_p), ("kpool", c_void_p), ("vpool", c_void_p)])
+                   ("max_pages", c_int), ("q", c_void_p), ("kpool", c_void_p), ("vpool", c_void_p), ("k_split", c_int)])
 
 
 class DiffAttnArgs(C.Structure):
     """vlm_diff_attn_args (include/vlm_hip.h)"""
     _fields_ = ([(n, c_void_p) for n in ("q", "kpool", "vpool", "qb_start", "qb_count", "tok_seq", "tok_pos", "block_table")]
                 + [(n, c_int) for n in ("max_pages", "H", "KH", "D", "Dv")] + [("scale", c_float), ("window", c_int), ("keep", c_int)]
-                + [(n, c_float) for n in ("lam", "mult", "eps")] + [("out", c_void_p), ("ldo", C.c_long)])
+                + [(n, c_float) for n in ("lam", "mult", "eps")] + [("out", c_void_p), ("ldo", C.c_long), ("nsplit", c_int), ("part", c_void_p)])
 
 
 class HyperArgs(C.Structure):

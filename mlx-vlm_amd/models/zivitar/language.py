@@ -7,7 +7,7 @@ the serving dtype.  The embedding rows stand for all S streams until the first w
     lightning : fixed-decay matrix-state recurrence on silu(q), silu(k), silu(v), state fp32 per sequence; RMS norm over all heads of a
                 token with a weight, times sigmoid(g); W_o
     attention : short causal convolution over the packed [q | k | v] columns (projected values carried per sequence), rotate-half
-                positions on the first rot dims of every map, keys (fp32) and values into the paged caches - one kernel; differential
+                positions on the first rot dims of every map, keys (fp32 precision) and values into the paged caches - one kernel; differential
                 softmax attention inside a window that keeps the first tokens in view, difference normed per head - one kernel; W_o
     dense     : [gate | up] in one GEMM, clamped gated activation, W_down
 Final norm of the summed streams at the wanted rows, logits = cap tanh(scale (rows @ head^T) / cap).  A layer with `weights_of` uses
@@ -94,7 +94,8 @@ class LanguageModel(RaggedLanguageModel):
                 ns.window, ns.keep = L.window
                 ns.rot_dims, f, ns.amp = rotation(m.get("rot"))
                 ns.inv_freq = torch.from_numpy(f).to(dev) if f is not None else None
-                rows[(i, "k")] = (ns.G * 2 * ns.D, f32)                    # rotated keys, never rounded
+                # rotated keys: fp32, or two bf16 values per coordinate (the same bytes)
+                rows[(i, "k")] = (ops.diff_key_width(ns.G * 2, ns.D, T == torch.bfloat16), T)
                 rows[(i, "v")] = (ns.G * ns.Dv, T)
                 if ns.taps > 1:
                     aux[(i, "conv")] = (ns.taps - 1, ns.wproj.shape[0])

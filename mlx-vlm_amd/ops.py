@@ -961,11 +961,17 @@ def hyper_step(xin, S, y=None, mix=None, out=None, w_in=None, w=None, eps=1e-6, 
     return h if w is not None else None
 
 
+def diff_key_width(heads, D, split):
+    """width of a cached key row of `heads` key vectors of D: fp32 as they are, or (split, bf16 pool) hi and lo planes padded to 8"""
+    return heads * (2 * ((D + 7) & ~7) if split else D)
+
+
 def conv_qkv_rows(x, w, carry, offs, HQ, HK, D, NV, tok_seq, tok_pos, cu, slot, pos0, block_table, q, kpool, vpool, rot_dims=0,
                   inv_freq=None, amp=1.0):
     """Packed projection rows x [T, C] = [q | k | v] at columns offs -> short causal convolution (w [C, taps], None: none; carry
     fp32 [slots, taps - 1, C], moved to the end of the step's segments) -> rotate-half positions on the first rot_dims dimensions of the
-    HQ + HK heads of q and k (cos and sin times amp) -> q fp32 [T, HQ * D] and the paged pools (keys fp32, values in x's dtype)."""
+    HQ + HK heads of q and k (cos and sin times amp) -> q fp32 [T, HQ * D] and the paged pools (values in x's dtype; keys fp32 rows [HK * D],
+    or with a bf16 key pool of rows diff_key_width(HK, D) every coordinate as two bf16 values)."""
     _dev(x, w, carry, tok_seq, tok_pos, cu, slot, pos0, block_table, q, kpool, vpool, inv_freq)
     T, C_ = x.shape
     taps = w.shape[1] if w is not None else 0
@@ -973,14 +979,15 @@ def conv_qkv_rows(x, w, carry, offs, HQ, HK, D, NV, tok_seq, tok_pos, cu, slot, 
         raise _lib.VlmHipError("conv_qkv_rows: one filter per packed column and a value pool, both of the rows' dtype, expected")
     if taps > 1 and (carry is None or carry.dtype != torch.float32 or tuple(carry.shape[1:]) != (taps - 1, C_)):
         raise _lib.VlmHipError("conv_qkv_rows: fp32 carry [slots, taps - 1, columns] expected")
-    if q.dtype != torch.float32 or kpool.dtype != torch.float32 or q.numel() != T * HQ * D or kpool.shape[-1] != HK * D or vpool.shape[-1] != NV:
-        raise _lib.VlmHipError("conv_qkv_rows: fp32 q rows [T, HQ * D], key pool [.., HK * D], value pool [.., NV] expected")
+    split = kpool.dtype == torch.bfloat16
+    if q.dtype != torch.float32 or q.numel() != T * HQ * D or kpool.shape[-1] != diff_key_width(HK, D, split) or vpool.shape[-1] != NV:
+        raise _lib.VlmHipError("conv_qkv_rows: fp32 q rows [T, HQ * D], a key pool of HK heads, value pool [.., NV] expected")
     a = _lib.ConvQkvArgs()
     a.x, a.ldx, a.w, a.carry, a.C, a.taps = _p(x), x.stride(0), _p(w), _p(carry), int(C_), int(taps)
     a.qoff, a.koff, a.voff = (int(o) for o in offs)
     a.HQ, a.HK, a.D, a.NV, a.rot_dims, a.inv_freq, a.amp = int(HQ), int(HK), int(D), int(NV), int(rot_dims), _p(inv_freq), float(amp)
     a.tok_seq, a.tok_pos, a.block_table, a.max_pages = _p(tok_seq), _p(tok_pos), _p(block_table), block_table.shape[1]
-    a.q, a.kpool, a.vpool = _p(q), _p(kpool), _p(vpool)
+    a.q, a.kpool, a.vpool, a.k_split = _p(q), _p(kpool), _p(vpool), int(split)
     check(_lib.lib().vlm_conv_qkv_rows(C.byref(a), T, _f32(x), _stream()), "conv_qkv_rows")
     if taps > 1:
         b = _lib.ShortConvArgs()
@@ -991,9 +998,9 @@ def conv_qkv_rows(x, w, carry, offs, HQ, HK, D, NV, tok_seq, tok_pos, cu, slot, 
 
 
 def _diff_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window, keep):
-    if q.dtype != torch.float32 or kpool.dtype != torch.float32 or vpool.dtype != out.dtype or not q.is_contiguous():
-        raise _lib.VlmHipError("diff_attn: fp32 queries and keys, values and output of one dtype expected")
-    if kpool.shape[-1] != KH * 2 * D or vpool.shape[-1] != KH * Dv or q.numel() != tok_seq.numel() * H * 2 * D:
+    if q.dtype != torch.float32 or kpool.dtype != vpool.dtype or vpool.dtype != out.dtype or not q.is_contiguous():
+        raise _lib.VlmHipError("diff_attn: fp32 queries; keys, values and output of one dtype expected")
+    if kpool.shape[-1] != diff_key_width(KH * 2, D, kpool.dtype == torch.bfloat16) or vpool.shape[-1] != KH * Dv or q.numel() != tok_seq.numel() * H * 2 * D:
         raise _lib.VlmHipError("diff_attn: two maps of D per head in q and the key pool, Dv value columns per head")
     a = _lib.DiffAttnArgs()
     a.q, a.kpool, a.vpool, a.tok_seq, a.tok_pos, a.block_table = _p(q), _p(kpool), _p(vpool), _p(tok_seq), _p(tok_pos), _p(block_table)
@@ -1004,7 +1011,8 @@ def _diff_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv
 
 def diff_attn_blocks(q, kpool, vpool, qb_start, qb_count, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window=0,
                      keep=0):
-    """differential attention, prompt form: q fp32 [T, H * 2 * D], pools with rows [KH * 2 * D] / [KH * Dv], out [T, H * Dv];
+    """differential attention, prompt form: q fp32 [T, H * 2 * D], pools with rows
+    [diff_key_width(KH * 2, D)] / [KH * Dv] in the serving dtype, out [T, H * Dv];
     window > 0: a query reaches back window - 1 tokens and to the first `keep` tokens of its sequence"""
     _dev(q, kpool, vpool, qb_start, qb_count, tok_seq, tok_pos, block_table, out)
     a = _diff_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window, keep)
@@ -1013,10 +1021,18 @@ def diff_attn_blocks(q, kpool, vpool, qb_start, qb_count, tok_seq, tok_pos, bloc
     return out
 
 
-def diff_attn_rows(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window=0, keep=0):
-    """differential attention, decode form (one workgroup per token and group of heads that share a key / value head)"""
+def diff_attn_rows(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window=0, keep=0,
+                   nsplit=None):
+    """differential attention, decode form: one token and the heads that share a key / value head per workgroup; few such column
+    groups share their keys between several workgroups each (merged by a second kernel)"""
     _dev(q, kpool, vpool, tok_seq, tok_pos, block_table, out)
+    rows = tok_seq.numel()
+    groups = rows * KH * -(-(H // KH) // 16)
+    span = min(block_table.shape[1] * 64, window + keep if window > 0 else 1 << 30)             # keys a query can see
+    nsplit = max(1, min(256 // max(groups, 1), -(-span // 128), 32)) if nsplit is None else int(nsplit)
+    part = torch.empty(nsplit, H, rows, 2, Dv + 2, dtype=torch.float32, device=q.device) if nsplit > 1 else None
     a = _diff_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window, keep)
+    a.nsplit, a.part = nsplit, _p(part)
     check(_lib.lib().vlm_diff_attn_rows(C.byref(a), tok_seq.numel(), _f32(vpool), _stream()), "diff_attn_rows")
     return out
 

@@ -85,8 +85,11 @@ def test_weights_load_on_the_cpu_device_with_shape_checks_and_state_per_layer():
         lm.load_weights(dict(W, unused=torch.zeros(3)))                           # a tensor nobody asks for is left alone
         pool = lm.pool
         assert sorted(pool.rows) == sorted((r, n) for r in (1, 2, 4, 5, 6) for n in "kv")
-        assert pool.rows[(1, "k")].dtype == torch.float32 and pool.rows[(1, "v")].dtype == T
-        assert pool.rows[(1, "k")].shape == (5, PAGE, 2 * 2 * 12) and pool.rows[(4, "v")].shape == (5, PAGE, 2 * 20) and pool.rows[(6, "k")].shape == (5, PAGE, 12)
+        # keys: two maps per head, fp32 or two bf16 planes padded to 8
+        split = T == torch.bfloat16
+        assert pool.rows[(1, "k")].dtype == T and pool.rows[(1, "v")].dtype == T
+        assert pool.rows[(1, "k")].shape == (5, PAGE, 2 * 2 * (2 * 16 if split else 12)) and pool.rows[(6, "k")].shape == (5, PAGE, 2 * 2 * 8 if split else 12)
+        assert pool.rows[(4, "v")].shape == (5, PAGE, 2 * 20)
         assert sorted(pool.state) == [0, 3, 7] and pool.state[0].shape == (3, 3, 10, 14) and all(t.dtype == torch.float32 for t in pool.state.values())
         # packed projection rows: 4 * 2 * 12 | 2 * 2 * 12 | 2 * 20 ; carried: taps - 1 of them per sequence (none for one tap)
         assert sorted(pool.aux) == [(1, "conv"), (2, "conv"), (4, "conv")] and pool.aux[(1, "conv")].shape == (3, 2, 96 + 48 + 40)

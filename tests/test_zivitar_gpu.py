@@ -77,6 +77,24 @@ def _segments(lens, slots, pos0):
     return tok_seq, tok_pos, cu, torch.tensor(slots, dtype=i32).cuda(), torch.tensor(pos0, dtype=i32).cuda()
 
 
+def _split_rows(k, heads, D):
+    """fp32 key rows [.., heads * D] as a bf16 pool keeps them: per head hi = bf16(k) and lo = bf16(k - hi), each padded to 8 columns"""
+    D8 = (D + 7) & ~7
+    v = k.view(*k.shape[:-1], heads, D)
+    hi = v.to(torch.bfloat16)
+    out = torch.zeros(*k.shape[:-1], heads, 2, D8, dtype=torch.bfloat16)
+    out[..., 0, :D], out[..., 1, :D] = hi, (v - hi.float()).to(torch.bfloat16)
+    return out.reshape(*k.shape[:-1], heads * 2 * D8)
+
+
+def _joined_rows(pool, heads, D):
+    """what such a pool holds, in float64"""
+    if pool.dtype == torch.float32:
+        return pool.double()
+    v = pool.double().view(*pool.shape[:-1], heads, 2, (D + 7) & ~7)
+    return (v[..., 0, :D] + v[..., 1, :D]).reshape(*pool.shape[:-1], heads * D)
+
+
 # ------------------------------------------------------------------------------------------------ operators
 @pytest.mark.parametrize("S", [1, 2, 3, 5, 8])
 @pytest.mark.parametrize("D", [52, 51, 1280])
@@ -132,7 +150,8 @@ def test_convolved_rotated_rows_across_portions_pages_and_reused_slots(T, taps):
         seqs = {s: torch.randn(n, C + 8, generator=g).to(T) for s, n in ((0, 99), (2, 71), (1, 5))}
         carry = torch.full((3, taps - 1, C), float("nan")).cuda() if taps > 1 else None
         bt = (torch.randperm(6, generator=g).to(torch.int32) + 1).view(3, 2).contiguous()
-        kpool, vpool = torch.zeros(7, PAGE, HK * D).cuda(), torch.zeros(7, PAGE, NV, dtype=T).cuda()
+        kpool = torch.zeros(7, PAGE, ops.diff_key_width(HK, D, T == torch.bfloat16), dtype=T).cuda()
+        vpool = torch.zeros(7, PAGE, NV, dtype=T).cuda()
 
         def reference(x):
             y = O.causal_conv(x.double()[:, :C], w.double()) if taps else x.double()[:, :C]
@@ -157,10 +176,10 @@ def test_convolved_rotated_rows_across_portions_pages_and_reused_slots(T, taps):
         tol = 2e-5 if T == torch.float32 else 5e-3
         for s, x in seqs.items():
             q, k, v = want[s]
-            kp = kpool[bt[s].long()].reshape(-1, HK * D)[: len(x)].cpu().double()
+            kp = _joined_rows(kpool[bt[s].long()].cpu(), HK, D).reshape(-1, HK * D)[: len(x)]
             vp = vpool[bt[s].long()].reshape(-1, NV)[: len(x)].cpu().double()
             assert (torch.cat(got[s]).double() - q).abs().max() < 2e-5, s          # fp32 from the projected row on, whatever T is
-            assert (kp - k).abs().max() < 2e-5 and ((vp - v).abs() <= tol * (1e-2 + v.abs())).all(), s
+            assert ((kp - k).abs() <= 2e-5 + 2.0 ** -16 * k.abs()).all() and ((vp - v).abs() <= tol * (1e-2 + v.abs())).all(), s
         got[0], at[0] = [], 0                                                       # slot 0 again, from position 0
         launch([(0, 4)], {0: seqs[2]})
         assert (torch.cat(got[0]).double() - want[2][0][:4]).abs().max() < 2e-5
@@ -184,6 +203,8 @@ def test_differential_attention_against_dense_maps(dtype, D, Dv, Hh, G):
     q = torch.randn(42, Hh * 2 * D, generator=g)
     qb_start = torch.tensor([0, 16, 32, 37], dtype=torch.int32).cuda()
     qb_count = torch.tensor([16, 16, 5, 5], dtype=torch.int32).cuda()
+    pool = kpool if dtype == torch.float32 else _split_rows(kpool, G * 2, D)
+    kpool = _joined_rows(pool, G * 2, D)
     rows = {sq: (kpool[bt[sq].long()].reshape(-1, G, 2, D).double(), vpool[bt[sq].long()].reshape(-1, G, Dv).double()) for sq in (1, 2)}
     qd = q.double().view(42, Hh, 2, D)
     for window, keep, scale, lam, diff in ((0, 0, 1.0, 0.7, 0.6), (17, 0, 1.0, 0.3, 0.2), (17, 4, 2.0, 0.9, 0.5), (1025, 70, 0.5, 1.2, 0.8),
@@ -199,10 +220,11 @@ def test_differential_attention_against_dense_maps(dtype, D, Dv, Hh, G):
                 want[t, h] = O.rms(a[0] - lam * a[1], 1e-5) * (1.0 - diff)
         args = (tok_seq.cuda(), tok_pos.cuda(), bt.cuda(), Hh, G, D, Dv, scale, lam, 1.0 - diff, 1e-5)
         a, b = (torch.full((42, Hh * Dv + 8), float("nan"), dtype=dtype, device="cuda")[:, : Hh * Dv] for _ in range(2))
-        ops.diff_attn_rows(q.cuda(), kpool.cuda(), vpool.cuda(), *args, a, window=window, keep=keep)
-        ops.diff_attn_blocks(q.cuda(), kpool.cuda(), vpool.cuda(), qb_start, qb_count, *args, b, window=window, keep=keep)
+        ops.diff_attn_blocks(q.cuda(), pool.cuda(), vpool.cuda(), qb_start, qb_count, *args, b, window=window, keep=keep)
         tol = 1e-4 if dtype == torch.float32 else 2e-2                              # (the norm magnifies what the difference cancels)
-        assert (a.cpu().double().view(42, Hh, Dv) - want).abs().max() < tol, (window, keep)
+        for nsplit in (None, 1, 2, 7, 64):                                          # workgroups that share a column group's keys
+            ops.diff_attn_rows(q.cuda(), pool.cuda(), vpool.cuda(), *args, a, window=window, keep=keep, nsplit=nsplit)
+            assert (a.cpu().double().view(42, Hh, Dv) - want).abs().max() < tol, (window, keep, nsplit)
         assert (b.cpu().double().view(42, Hh, Dv) - want).abs().max() < tol, (window, keep)
 
 
