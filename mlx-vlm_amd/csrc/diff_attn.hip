@@ -171,8 +171,8 @@ __global__ __launch_bounds__(NW * 64) void diff_attn_kernel(vlm_diff_attn_args p
   const int D8 = (D + 7) & ~7, DPB = (D + 31) & ~31, QPB = DPB + 8;   // bf16 queries: [2][2][QC][QPB]
   float* qs = smem;                                      // queries times scale * log2(e)
   bf16_t* qb = reinterpret_cast<bf16_t*>(smem);
-  float* ml = qs + (F32 ? 2 * QC * QP : 2 * QC * QPB);   // [NW][2][QC][2]: running maximum and sum of every wave
-  float* os = ml + NW * 2 * QC * 2;                      // [2][QC][OP]
+  float* os = smem;                                      // [2][QC][OP], in the queries' place once every wave is through its keys
+  float* ml = smem + max(F32 ? 2 * QC * QP : 2 * QC * QPB, 2 * QC * OP);   // [NW][2][QC][2]: running maximum and sum of every wave
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r16 = lane & 15, g = lane >> 4;
   const int R = p.H / p.KH;
   // the workgroup's columns
@@ -393,32 +393,33 @@ __global__ __launch_bounds__(NW * 64) void diff_attn_kernel(vlm_diff_attn_args p
   }
 }
 
-// merge of the splits' partial results: grid (rows, H), one wave.  part: [split][H][rows][2 maps][Dv sums | maximum | sum]
+// merge of the splits' partial results: grid (rows, H), 4 waves (wave w: map w & 1, every other 64 value columns from 64 (w >> 1)).
+// part: [split][H][rows][2 maps][Dv sums | maximum | sum]
 template <typename T>
-__global__ __launch_bounds__(64) void diff_attn_merge_kernel(vlm_diff_attn_args p, int nsplit) {
+__global__ __launch_bounds__(256) void diff_attn_merge_kernel(vlm_diff_attn_args p, int nsplit) {
   extern __shared__ float sm[];                          // [2][Dv]
   const long t = blockIdx.x;
-  const int h = blockIdx.y, lane = threadIdx.x, Dv = p.Dv;
+  const int h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m = wave & 1, Dv = p.Dv;
   const long step = (long)p.H * gridDim.x * 2 * (Dv + 2);
-  const float* base = p.part + ((long)h * gridDim.x + t) * 2 * (Dv + 2);
+  const float* q = p.part + (((long)h * gridDim.x + t) * 2 + m) * (Dv + 2);
+  const float M_mine = lane < nsplit ? q[lane * step + Dv] : -INFINITY, l_mine = lane < nsplit ? q[lane * step + Dv + 1] : 0.f;
+  const float M = wave_max(M_mine);
+  const float f_mine = M == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(M_mine - M);
+  const float l = wave_sum(l_mine * f_mine), inv = l > 0.f ? 1.f / l : 0.f;
+  for (int c0 = 64 * (wave >> 1); c0 < Dv; c0 += 128) {  // (whole waves: the shuffles below need every lane)
+    const int c = min(c0 + lane, Dv - 1);
+    float a = 0.f;
+    for (int z0 = 0; z0 < nsplit; z0 += 8) {             // eight loads in flight; splits past the last one count for nothing
+      float v[8];
 #pragma unroll
-  for (int m = 0; m < 2; ++m) {
-    const float* q = base + m * (Dv + 2);
-    const float M_mine = lane < nsplit ? q[lane * step + Dv] : -INFINITY, l_mine = lane < nsplit ? q[lane * step + Dv + 1] : 0.f;
-    const float M = wave_max(M_mine);
-    const float f_mine = M == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(M_mine - M);
-    const float l = wave_sum(l_mine * f_mine), inv = l > 0.f ? 1.f / l : 0.f;
-    for (int c0 = 0; c0 < Dv; c0 += 64) {                // (whole waves: the shuffles below need every lane)
-      const int c = c0 + lane;
-      float a = 0.f;
-      for (int z = 0; z < nsplit; ++z) {
-        const float f = __shfl(f_mine, z);
-        if (c < Dv) a = fmaf(f, q[z * step + c], a);
-      }
-      if (c < Dv) sm[m * Dv + c] = a * inv;
+      for (int i = 0; i < 8; ++i) v[i] = q[min(z0 + i, nsplit - 1) * step + c];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) a = fmaf(__shfl(f_mine, min(z0 + i, 63)) * (z0 + i < nsplit ? 1.f : 0.f), v[i], a);
     }
+    if (c0 + lane < Dv) sm[m * Dv + c] = a * inv;
   }
   __syncthreads();
+  if (wave) return;
   const float* o1 = sm;
   const float* o2 = sm + Dv;
   difference_store<T>([&](int i) { return o1[i]; }, [&](int i) { return o2[i]; }, Dv, p.lambda, p.eps, p.mult, lane & 15, lane < 16,
@@ -427,7 +428,8 @@ __global__ __launch_bounds__(64) void diff_attn_merge_kernel(vlm_diff_attn_args 
 
 size_t lds_bytes(const vlm_diff_attn_args& a, int NB, int NW, bool f32) {
   const size_t q = f32 ? (size_t)2 * QC * (((a.D + 15) & ~15) + 4) : (size_t)2 * QC * (((a.D + 31) & ~31) + 8);
-  return (q + (size_t)NW * 2 * QC * 2 + (size_t)2 * QC * (NB * 16 + 4)) * sizeof(float);
+  const size_t o = (size_t)2 * QC * (NB * 16 + 4);
+  return ((q > o ? q : o) + (size_t)NW * 2 * QC * 2) * sizeof(float);
 }
 
 template <typename T, int NW>
@@ -470,8 +472,8 @@ extern "C" int vlm_diff_attn_rows(const vlm_diff_attn_args* a, int rows, int dty
   const int rc = dtype ? launch<float, 4>(*a, grid, 1, hpb, st) : launch<bf16_t, 4>(*a, grid, 1, hpb, st);
   if (rc || nsplit == 1) return rc;
   const size_t lds = (size_t)2 * a->Dv * sizeof(float);
-  if (dtype) hipLaunchKernelGGL(diff_attn_merge_kernel<float>, dim3(rows, a->H), dim3(64), lds, st, *a, nsplit);
-  else hipLaunchKernelGGL(diff_attn_merge_kernel<bf16_t>, dim3(rows, a->H), dim3(64), lds, st, *a, nsplit);
+  if (dtype) hipLaunchKernelGGL(diff_attn_merge_kernel<float>, dim3(rows, a->H), dim3(256), lds, st, *a, nsplit);
+  else hipLaunchKernelGGL(diff_attn_merge_kernel<bf16_t>, dim3(rows, a->H), dim3(256), lds, st, *a, nsplit);
   VLM_CHECK_LAUNCH();
   return VLM_OK;
 }

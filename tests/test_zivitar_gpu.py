@@ -186,7 +186,7 @@ def test_convolved_rotated_rows_across_portions_pages_and_reused_slots(T, taps):
 
 
 @pytest.mark.parametrize("D,Dv,Hh,G", [(12, 20, 6, 2), (16, 16, 2, 2), (6, 33, 3, 1), (40, 72, 20, 1), (64, 128, 6, 2), (72, 136, 4, 2), (1, 1, 1, 1),
-                                       (18, 256, 2, 1)])
+                                       (18, 256, 2, 1), (256, 256, 1, 1), (320, 24, 2, 1)])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_differential_attention_against_dense_maps(dtype, D, Dv, Hh, G):
     """two sequences at different offsets on scattered pages (one 1890 tokens deep), windows with and without kept tokens, both forms"""
