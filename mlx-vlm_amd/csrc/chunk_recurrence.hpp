@@ -7,4 +7,4 @@
 #define VLM_CHUNK_MIN 17          // segments of at least this many tokens take the chunk-parallel form
 
 // the raw read-outs and states of the segments of more than max_len tokens (the other segments are left alone)
-int vlm_chunk_recurrence(const vlm_recurrence_args* a, int nseg, int ntok, int max_len, int dtype, hipStream_t st);
+__attribute__((visibility("hidden"))) int vlm_chunk_recurrence(const vlm_recurrence_args* a, int nseg, int ntok, int max_len, int dtype, hipStream_t st);
