@@ -626,16 +626,39 @@ int vlm_latent_kv_write(const void* d, long ldd, const void* w, int R, int Dr, c
                         int dtype, void* stream);
 /* rot_half (both functions above and below): 0 = the rotated pairs are (2 i, 2 i + 1), 1 = (i, i + Dr / 2).  ABI v11. */
 int vlm_rope_pairs_rows(const void* q, long ldq, long head_stride, int H, int Dr, const void* inv_freq, const void* tok_pos, void* out,
-                        long ldo, long out_head_stride, int rot_half, int rows, int dtype, void* stream);
-/* window > 0 (ABI v11): query i sees the keys j with 0 <= i - j < window; <= 0: every j <= i */
+                        long ldo, long out_head_stride, int rot_half, float amp, int rows, int dtype, void* stream);
+/* ABI v14: amp: a factor on cos and sin (above and below); vlm_latent_kv_write with it, and with dq the RMS norm of the query's own latent
+ * (T rows [Rq] at lddq -> cq) in the same launch. */
+typedef struct vlm_latent_prep_args {
+  const void* d;                        /* T rows [R + Dr] at ldd */
+  long ldd;
+  const void* w;                        /* T [R] */
+  int R, Dr;
+  const float* inv_freq;
+  float amp;
+  int rot_half;
+  const int *tok_seq, *tok_pos, *block_table;
+  int max_pages;
+  void* pool;                           /* T [pages][64][R + Dr] */
+  float eps;
+  const void* dq;                       /* T rows [Rq] at lddq, or NULL */
+  long lddq;
+  const void* wq;                       /* T [Rq] */
+  int Rq;
+  void* cq;                             /* T rows [Rq] at ldcq */
+  long ldcq;
+} vlm_latent_prep_args;
+int vlm_latent_prep_rows(const vlm_latent_prep_args* a, int rows, int dtype, void* stream);
+/* window > 0 (ABI v11): query i sees the keys j with 0 <= i - j < window; <= 0: every j <= i
+ * sink (ABI v14): fp32 [H] or NULL: the softmax's denominator also contains exp(sink[h]) */
 int vlm_latent_attn(const void* q, const void* pool, const void* tok_seq, const void* tok_pos, const void* block_table, int max_pages,
-                    int H, int R, int Dr, float scale, int window, const void* gate, long ldgate, void* out, int rows, int dtype,
-                    void* stream);
+                    int H, int R, int Dr, float scale, int window, const void* sink, const void* gate, long ldgate, void* out, int rows,
+                    int dtype, void* stream);
 /* the prompt form: query blocks (first token, count <= 16, all of one sequence and consecutive) x heads, key tiles through LDS;
  * R <= 512.  Same results as vlm_latent_attn up to summation order. */
 int vlm_latent_attn_blocks(const void* q, const void* pool, const void* qb_start, const void* qb_count, int nblocks, const void* tok_seq,
                            const void* tok_pos, const void* block_table, int max_pages, int H, int R, int Dr, float scale, int window,
-                           const void* gate, long ldgate, void* out, int dtype, void* stream);
+                           const void* sink, const void* gate, long ldgate, void* out, int dtype, void* stream);
 
 /* csrc/moe.hip */
 int vlm_moe_route(const void* logits, int T, int E, int top, void* gate, void* idx, void* wgt, void* stream);
@@ -655,8 +678,15 @@ int vlm_moe_route_scored(const void* logits, int T, int E, int top, int groups, 
 int vlm_moe_route_sigmoid(const void* logits, long ldz, int T, int E, int top, int groups, int keep, int group_top, const void* correction,
                           int normalise, float scale, int extra, void* extra_out, void* gate, void* idx, void* wgt, void* stream);
 /* ABI v13: act 3 = clamped gate: g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit). */
+/* ABI v14: act 4 = relu; gbias / ubias (T [dim] or NULL, without a route table): added to g and u first. */
 int vlm_glu_rows(const void* g, long ldg, const void* u, long ldu, const void* route, int E, int ff, int estride, int act, float limit,
-                 void* out, long ldo, int rows, int dim, int dtype, void* stream);
+                 const void* gbias, const void* ubias, void* out, long ldo, int rows, int dim, int dtype, void* stream);
+/* ABI v14.  Router logits and choice in one kernel: z = h W^T (T rows [D] at ldh, T [E][D] at ldw, fp32 sums), s = softmax(z) over all E
+ * columns, the `top` largest of s + correction (fp32 [E] or NULL; lowest index wins a tie) keep the weight s.  gate: fp32 [T][E - identity],
+ * 0 where not chosen; the last `identity` columns stand for experts that hand their input on: the sum of their weights goes to
+ * ident fp32 [T].  E <= 256. */
+int vlm_moe_router_softmax(const void* h, long ldh, const void* w, long ldw, int D, int T, int E, int top, int identity,
+                           const void* correction, void* gate, void* ident, int dtype, void* stream);
 int vlm_moe_relu2_gate(const void* up, long ldu, const void* gate, int E, int ff, int shared, void* out, long ldo, int rows, int dtype,
                        void* stream);
 
@@ -674,6 +704,29 @@ int vlm_relu2_rows(const void* in, long ldi, void* out, long ldo, int rows, int 
  * T is (a reader that goes on in fp32, e.g. a short convolution over the normed rows). */
 int vlm_scaled_add_rms(void* x, const void* y, long ldy, float mult, const void* y2, long ldy2, float mult2, const void* w, float w_offset,
                        void* h, long ldh, int h_f32, int rows, int D, float eps, int dtype, void* stream);
+
+/* ABI v14.  The residual step of a sublayer that is normed before and after, fused with the next reader's norm:
+ *   r = y[t] (+ bias) (+ pass[t] * src[t])     x[t] <- (init ? 0 : x[t]) + mult * rms(r) * wy     h[t] = rms(x[t]) * w, or T(x[t]) without w */
+typedef struct vlm_sandwich_args {
+  float* x;                             /* fp32 [rows][D] */
+  int init;                             /* 1: x is written, not read */
+  const int* ids;                       /* [rows] or NULL: read row ids[t] of y (vocab rows) instead of row t */
+  int vocab;
+  const void* y;                        /* T rows [D] at ldy */
+  long ldy;
+  const void* bias;                     /* T [D] or NULL */
+  const float* pass;                    /* [rows] or NULL */
+  const void* src;                      /* T rows [D] at ldsrc */
+  long ldsrc;
+  const void* wy;                       /* T [D] */
+  float mult;
+  const void* w;                        /* T [D] or NULL */
+  void* h;                              /* T rows [D] at ldh or NULL */
+  long ldh;
+  int D;
+  float eps;
+} vlm_sandwich_args;
+int vlm_sandwich_step(const vlm_sandwich_args* a, int rows, int dtype, void* stream);
 
 /* csrc/delta_rule.hip: delta-rule recurrences (the update reads the old state), state fp32 [slots][H][D][Dv].
  * Prepare passes write fp32 rows; the scan + finish take them.  Segments as in vlm_linear_recurrence. */
@@ -832,6 +885,50 @@ typedef struct vlm_diff_attn_args {
 } vlm_diff_attn_args;
 int vlm_diff_attn_blocks(const vlm_diff_attn_args* a, int nblocks, int dtype, void* stream);
 int vlm_diff_attn_rows(const vlm_diff_attn_args* a, int rows, int dtype, void* stream);
+
+/* csrc/grouped_attn.hip (ABI v14).  Packed projection rows -> q (x + bias, RMS norm over all heads at once, weight, times
+ * 1 + temp_coef * ln(floor((pos + 1) / temp_every) + 1)) as dense fp32 rows; k likewise without the multiplier into its paged pool (fp32 rows
+ * [HK * D]; with k_split as bf16 pairs hi + lo, [HK][2][D8], D8 = D rounded up to 8); v + bias into its paged pool, with vother mixed
+ * with the values another pool of the same paging holds for the token: (1 - mix) v + mix v_other. */
+typedef struct vlm_qkv_rownorm_args {
+  const void* x;                        /* T rows at ldx */
+  long ldx;
+  int qoff, koff, voff, HQ, HK, D, NV;  /* first columns of the parts, heads, value columns */
+  const void *qbias, *kbias, *vbias;    /* T or NULL */
+  const void *qw, *kw;                  /* T [HQ * D], [HK * D] */
+  float eps, temp_coef;
+  int temp_every;                       /* 0: no multiplier */
+  const int *tok_seq, *tok_pos, *block_table;
+  int max_pages;
+  float* q;
+  void *kpool, *vpool;
+  const void* vother;                   /* T [pages][64][NV] or NULL */
+  float mix;
+  int k_split;
+} vlm_qkv_rownorm_args;
+int vlm_qkv_rownorm_rows(const vlm_qkv_rownorm_args* a, int rows, int dtype, void* stream);
+
+/* Grouped-head softmax attention on the matrix cores: s_ij = (q_i . k_j) scale - slope_h (i - j) for 0 <= i - j < window (window <= 0: every
+ * j <= i), o_i = sum_j exp(s_ij) v_j / (exp(sink_h) + sum_j exp(s_ij)) * sigmoid(gate_ih).  Forms as in vlm_diff_attn_blocks / _rows. */
+typedef struct vlm_grouped_attn_args {
+  const float* q;                       /* [tokens][H][D] */
+  const void* kpool;                    /* dtype fp32: fp32 [pages][64][KH][D]; bf16: [pages][64][KH][2 (hi, lo)][D8], padding zero */
+  const void* vpool;                    /* T [pages][64][KH][Dv] */
+  const int *qb_start, *qb_count;       /* _blocks only */
+  const int *tok_seq, *tok_pos, *block_table;
+  int max_pages, H, KH, D, Dv;
+  float scale;
+  int window;
+  const float *slope, *sink;            /* fp32 [H] or NULL */
+  const void* gate;                     /* T rows [H] at ldgate or NULL */
+  long ldgate;
+  void* out;                            /* T rows [H * Dv] at ldo */
+  long ldo;
+  int nsplit;                           /* _rows: workgroups that share a column group's keys (0 / 1: one; at most 64) */
+  float* part;                          /* nsplit > 1: scratch fp32 [nsplit][H][rows][Dv + 2] */
+} vlm_grouped_attn_args;
+int vlm_grouped_attn_blocks(const vlm_grouped_attn_args* a, int nblocks, int dtype, void* stream);
+int vlm_grouped_attn_rows(const vlm_grouped_attn_args* a, int rows, int dtype, void* stream);
 
 /* csrc/hyper_stream.hip (ABI v13): S residual streams per token, fp32 [rows][S][D], written and read in one pass:
  *   x'_t = sum_s mix[s][t] x_s + out[t] y  (y NULL: streams as they are)      h = rms(sum_t in[t] x'_t) * w  (w NULL: no read;

@@ -158,6 +158,37 @@ class DiffAttnArgs(C.Structure):
                 + [(n, c_float) for n in ("lam", "mult", "eps")] + [("out", c_void_p), ("ldo", C.c_long), ("nsplit", c_int), ("part", c_void_p)])
 
 
+class LatentPrepArgs(C.Structure):
+    """vlm_latent_prep_args (include/vlm_hip.h)"""
+    _fields_ = [("d", c_void_p), ("ldd", C.c_long), ("w", c_void_p), ("R", c_int), ("Dr", c_int), ("inv_freq", c_void_p), ("amp", c_float),
+                ("rot_half", c_int), ("tok_seq", c_void_p), ("tok_pos", c_void_p), ("block_table", c_void_p), ("max_pages", c_int),
+                ("pool", c_void_p), ("eps", c_float), ("dq", c_void_p), ("lddq", C.c_long), ("wq", c_void_p), ("Rq", c_int), ("cq", c_void_p),
+                ("ldcq", C.c_long)]
+
+
+class SandwichArgs(C.Structure):
+    """vlm_sandwich_args (include/vlm_hip.h)"""
+    _fields_ = [("x", c_void_p), ("init", c_int), ("ids", c_void_p), ("vocab", c_int), ("y", c_void_p), ("ldy", C.c_long), ("bias", c_void_p),
+                ("pass_", c_void_p), ("src", c_void_p), ("ldsrc", C.c_long), ("wy", c_void_p), ("mult", c_float), ("w", c_void_p),
+                ("h", c_void_p), ("ldh", C.c_long), ("D", c_int), ("eps", c_float)]
+
+
+class QkvRownormArgs(C.Structure):
+    """vlm_qkv_rownorm_args (include/vlm_hip.h)"""
+    _fields_ = ([("x", c_void_p), ("ldx", C.c_long)] + [(n, c_int) for n in ("qoff", "koff", "voff", "HQ", "HK", "D", "NV")]
+                + [(n, c_void_p) for n in ("qbias", "kbias", "vbias", "qw", "kw")] + [("eps", c_float), ("temp_coef", c_float), ("temp_every", c_int)]
+                + [(n, c_void_p) for n in ("tok_seq", "tok_pos", "block_table")] + [("max_pages", c_int)]
+                + [(n, c_void_p) for n in ("q", "kpool", "vpool", "vother")] + [("mix", c_float), ("k_split", c_int)])
+
+
+class GroupedAttnArgs(C.Structure):
+    """vlm_grouped_attn_args (include/vlm_hip.h)"""
+    _fields_ = ([(n, c_void_p) for n in ("q", "kpool", "vpool", "qb_start", "qb_count", "tok_seq", "tok_pos", "block_table")]
+                + [(n, c_int) for n in ("max_pages", "H", "KH", "D", "Dv")] + [("scale", c_float), ("window", c_int)]
+                + [(n, c_void_p) for n in ("slope", "sink", "gate")] + [("ldgate", C.c_long), ("out", c_void_p), ("ldo", C.c_long),
+                                                                        ("nsplit", c_int), ("part", c_void_p)])
+
+
 class HyperArgs(C.Structure):
     """vlm_hyper_args (include/vlm_hip.h)"""
     _fields_ = [("xin", c_void_p), ("xin_tok", C.c_long), ("xin_stream", C.c_long), ("xout", c_void_p), ("y", c_void_p), ("ldy", C.c_long),
@@ -266,14 +297,20 @@ SIGNATURES = {
     "vlm_latent_kv_write": (c_int, [c_void_p, C.c_long, c_void_p, c_int, c_int] + [c_void_p] * 4 + [c_int, c_void_p, c_float, c_int,
                                     c_int, c_int, c_void_p]),
     "vlm_rope_pairs_rows": (c_int, [c_void_p, C.c_long, C.c_long, c_int, c_int, c_void_p, c_void_p, c_void_p, C.c_long, C.c_long,
-                                    c_int, c_int, c_int, c_void_p]),
-    "vlm_latent_attn": (c_int, [c_void_p] * 5 + [c_int] * 4 + [c_float, c_int, c_void_p, C.c_long, c_void_p, c_int, c_int, c_void_p]),
-    "vlm_latent_attn_blocks": (c_int, [c_void_p] * 4 + [c_int] + [c_void_p] * 3 + [c_int] * 4 + [c_float, c_int, c_void_p, C.c_long,
+                                    c_int, c_float, c_int, c_int, c_void_p]),
+    "vlm_latent_prep_rows": (c_int, [P(LatentPrepArgs), c_int, c_int, c_void_p]),
+    "vlm_latent_attn": (c_int, [c_void_p] * 5 + [c_int] * 4 + [c_float, c_int, c_void_p, c_void_p, C.c_long, c_void_p, c_int, c_int, c_void_p]),
+    "vlm_latent_attn_blocks": (c_int, [c_void_p] * 4 + [c_int] + [c_void_p] * 3 + [c_int] * 4 + [c_float, c_int, c_void_p, c_void_p, C.c_long,
                                        c_void_p, c_int, c_void_p]),
+    "vlm_sandwich_step": (c_int, [P(SandwichArgs), c_int, c_int, c_void_p]),
+    "vlm_qkv_rownorm_rows": (c_int, [P(QkvRownormArgs), c_int, c_int, c_void_p]),
+    "vlm_grouped_attn_blocks": (c_int, [P(GroupedAttnArgs), c_int, c_int, c_void_p]),
+    "vlm_grouped_attn_rows": (c_int, [P(GroupedAttnArgs), c_int, c_int, c_void_p]),
+    "vlm_moe_router_softmax": (c_int, [c_void_p, C.c_long, c_void_p, C.c_long] + [c_int] * 5 + [c_void_p] * 3 + [c_int, c_void_p]),
     "vlm_moe_route": (c_int, [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p]),
     "vlm_moe_route_scored": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_void_p]),
-    "vlm_glu_rows": (c_int, [c_void_p, C.c_long, c_void_p, C.c_long, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p, C.c_long, c_int,
-                             c_int, c_int, c_void_p]),
+    "vlm_glu_rows": (c_int, [c_void_p, C.c_long, c_void_p, C.c_long, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, C.c_long,
+                             c_int, c_int, c_int, c_void_p]),
     "vlm_conv_qkv_rows": (c_int, [P(ConvQkvArgs), c_int, c_int, c_void_p]),
     "vlm_diff_attn_blocks": (c_int, [P(DiffAttnArgs), c_int, c_int, c_void_p]),
     "vlm_diff_attn_rows": (c_int, [P(DiffAttnArgs), c_int, c_int, c_void_p]),

@@ -19,6 +19,9 @@
 //                            sequence's first token
 // A sliding window (window > 0) limits query i to the keys j with 0 <= i - j < window; tiles still sit at multiples of their
 // size counted from the sequence's first token and start at the tile that holds the window's edge.
+// A sink (fp32 [H]) adds exp(sink_h) to the softmax's denominator: a learned number per head without key and value, which is not scaled.
+//   vlm_latent_prep_rows     vlm_latent_kv_write with a factor `amp` on cos and sin, and, for designs whose queries pass through a latent
+//                            of their own, that latent's RMS norm (d_q * rsqrt(mean(d_q^2) + eps) * w_q -> T rows) in the same launch
 // Scores, softmax and the weighted sum are fp32.  dtype: 0 = bf16, 1 = fp32 for the T-typed pointers.
 #include "common.hpp"
 #include "../../include/vlm_hip.h"
@@ -38,9 +41,25 @@ template <typename T>
 __global__ __launch_bounds__(256) void latent_kv_write_kernel(const T* __restrict__ d, long ldd, const T* __restrict__ w, int R, int Dr,
                                                               const float* __restrict__ inv_freq, const int* __restrict__ tok_seq,
                                                               const int* __restrict__ tok_pos, const int* __restrict__ block_table,
-                                                              int max_pages, T* __restrict__ pool, float eps, int rot_half) {
+                                                              int max_pages, T* __restrict__ pool, float eps, int rot_half, float amp,
+                                                              const T* __restrict__ dq, long lddq, const T* __restrict__ wq, int Rq,
+                                                              T* __restrict__ cq, long ldcq) {
   __shared__ float red[4];
   const long t = blockIdx.x;
+  if (blockIdx.y == 1) {                                  // the query's latent: normed rows
+    const T* qr = dq + t * lddq;
+    float s = 0.f;
+    for (int i = threadIdx.x; i < Rq; i += 256) {
+      const float v = ld_f(qr + i);
+      s += v * v;
+    }
+    s = wave_sum(s);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = s;
+    __syncthreads();
+    const float r = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)Rq + eps);
+    for (int i = threadIdx.x; i < Rq; i += 256) st_f(cq + t * ldcq + i, ld_f(qr + i) * r * ld_f(wq + i));
+    return;
+  }
   const T* row = d + t * ldd;
   const int pos = tok_pos[t];
   const int page = block_table[(long)tok_seq[t] * max_pages + pos / PAGE];
@@ -61,6 +80,8 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(const T* __restric
     const float u = ld_f(row + R + i0), v = ld_f(row + R + i1);
     float sn, cs;
     sincosf((float)pos * inv_freq[i], &sn, &cs);
+    sn *= amp;
+    cs *= amp;
     st_f(dst + R + i0, u * cs - v * sn);
     st_f(dst + R + i1, v * cs + u * sn);
   }
@@ -70,7 +91,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void rope_pairs_rows_kernel(const T* __restrict__ q, long ldq, long head_stride, int H, int Dr,
                                                               const float* __restrict__ inv_freq, const int* __restrict__ tok_pos,
                                                               float* __restrict__ out, long ldo, long out_head_stride, int rows,
-                                                              int rot_half) {
+                                                              int rot_half, float amp) {
   const long i = (long)blockIdx.x * 256 + threadIdx.x;
   const int hp = Dr / 2;
   if (i >= (long)rows * H * hp) return;
@@ -81,6 +102,8 @@ __global__ __launch_bounds__(256) void rope_pairs_rows_kernel(const T* __restric
   const float u = ld_f(src + i0), v = ld_f(src + i1);
   float sn, cs;
   sincosf((float)tok_pos[t] * inv_freq[pi], &sn, &cs);
+  sn *= amp;
+  cs *= amp;
   float* dst = out + t * ldo + (long)h * out_head_stride;
   dst[i0] = u * cs - v * sn;
   dst[i1] = v * cs + u * sn;
@@ -91,7 +114,7 @@ template <typename T, int NACC>
 __global__ __launch_bounds__(256) void latent_attn_kernel(const float* __restrict__ q, const T* __restrict__ pool,
                                                           const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
                                                           const int* __restrict__ block_table, int max_pages, int H, int R, int Dr,
-                                                          float scale, int window, const T* __restrict__ gate, long ldgate,
+                                                          float scale, int window, const float* __restrict__ sink, const T* __restrict__ gate, long ldgate,
                                                           float* __restrict__ out) {
   extern __shared__ float smem[];
   const int Dk = R + Dr;
@@ -150,7 +173,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const float* __restric
     }
     __syncthreads();
   }
-  float gsc = 1.f / l_run;
+  float gsc = 1.f / (sink ? l_run + expf(sink[h] - m_run) : l_run);
   if (gate) gsc *= 1.f / (1.f + expf(-ld_f(gate + t * ldgate + h)));
 #pragma unroll
   for (int a = 0; a < NACC; ++a) {
@@ -183,7 +206,8 @@ __global__ __launch_bounds__(256) void latent_attn_block_kernel(const float* __r
                                                                 const int* __restrict__ qb_start, const int* __restrict__ qb_count,
                                                                 const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
                                                                 const int* __restrict__ block_table, int max_pages, int H, int R,
-                                                                int Dr, float scale, int window, const T* __restrict__ gate,
+                                                                int Dr, float scale, int window, const float* __restrict__ sink,
+                                                                const T* __restrict__ gate,
                                                                 long ldgate, float* __restrict__ out) {
   extern __shared__ float smem[];
   const int Dk = R + Dr, DP = (Dk + 7) & ~7, KP = DP + 4;
@@ -300,7 +324,7 @@ __global__ __launch_bounds__(256) void latent_attn_block_kernel(const float* __r
 #pragma unroll
   for (int a = 0; a < QB; ++a) {
     if (a >= nq) break;
-    float gsc = 1.f / lrun[a];
+    float gsc = 1.f / (sink ? lrun[a] + expf(sink[h] - mrun[a]) : lrun[a]);
     if (gate) gsc *= 1.f / (1.f + expf(-ld_f(gate + (long)(t0 + a) * ldgate + h)));
 #pragma unroll
     for (int b = 0; b < NACC; ++b)
@@ -320,7 +344,8 @@ template <typename T>
 __global__ __launch_bounds__(256) void latent_attn_row_vec_kernel(const float* __restrict__ q, const T* __restrict__ pool,
                                                                   const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
                                                                   const int* __restrict__ block_table, int max_pages, int H, int R,
-                                                                  int Dr, float scale, int window, const T* __restrict__ gate,
+                                                                  int Dr, float scale, int window, const float* __restrict__ sink,
+                                                                const T* __restrict__ gate,
                                                                   long ldgate, float* __restrict__ out) {
   extern __shared__ __align__(16) float smem[];
   const int Dk = R + Dr;
@@ -408,7 +433,7 @@ __global__ __launch_bounds__(256) void latent_attn_row_vec_kernel(const float* _
 #pragma unroll
   for (int i = 0; i < 8; ++i) part[tid * 8 + i] = acc[i];
   __syncthreads();
-  float gsc = 1.f / l_run;
+  float gsc = 1.f / (sink ? l_run + expf(sink[h] - m_run) : l_run);
   if (gate) gsc *= 1.f / (1.f + expf(-ld_f(gate + t * ldgate + h)));
   for (int c = tid; c < R; c += 256) {
     float o = 0.f;
@@ -419,45 +444,54 @@ __global__ __launch_bounds__(256) void latent_attn_row_vec_kernel(const float* _
 
 }  // namespace
 
-extern "C" int vlm_latent_kv_write(const void* d, long ldd, const void* w, int R, int Dr, const void* inv_freq, const void* tok_seq,
-                                   const void* tok_pos, const void* block_table, int max_pages, void* pool, float eps, int rot_half,
-                                   int rows, int dtype, void* stream) {
-  if (!d || !w || !tok_seq || !tok_pos || !block_table || !pool || R <= 0 || Dr < 0 || (Dr & 1) || (Dr && !inv_freq) ||
-      ldd < R + Dr || max_pages <= 0 || rows < 0)
+extern "C" int vlm_latent_prep_rows(const vlm_latent_prep_args* a, int rows, int dtype, void* stream) {
+  if (!a || !a->d || !a->w || !a->tok_seq || !a->tok_pos || !a->block_table || !a->pool || a->R <= 0 || a->Dr < 0 || (a->Dr & 1) ||
+      (a->Dr && !a->inv_freq) || a->ldd < a->R + a->Dr || a->max_pages <= 0 || rows < 0 ||
+      (a->dq && (!a->wq || !a->cq || a->Rq <= 0 || a->lddq < a->Rq || a->ldcq < a->Rq)))
     return VLM_ERR_ARG;
   if (rows == 0) return VLM_OK;
   hipStream_t st = (hipStream_t)stream;
-  if (dtype)
-    hipLaunchKernelGGL(latent_kv_write_kernel<float>, dim3(rows), dim3(256), 0, st, (const float*)d, ldd, (const float*)w, R, Dr,
-                       (const float*)inv_freq, (const int*)tok_seq, (const int*)tok_pos, (const int*)block_table, max_pages,
-                       (float*)pool, eps, rot_half);
-  else
-    hipLaunchKernelGGL(latent_kv_write_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, (const bf16_t*)d, ldd, (const bf16_t*)w, R, Dr,
-                       (const float*)inv_freq, (const int*)tok_seq, (const int*)tok_pos, (const int*)block_table, max_pages,
-                       (bf16_t*)pool, eps, rot_half);
+  const dim3 grid(rows, a->dq ? 2 : 1);
+#define GO(T)                                                                                                                     \
+  hipLaunchKernelGGL(latent_kv_write_kernel<T>, grid, dim3(256), 0, st, (const T*)a->d, a->ldd, (const T*)a->w, a->R, a->Dr, a->inv_freq, \
+                     a->tok_seq, a->tok_pos, a->block_table, a->max_pages, (T*)a->pool, a->eps, a->rot_half, a->amp, (const T*)a->dq,     \
+                     a->lddq, (const T*)a->wq, a->Rq, (T*)a->cq, a->ldcq)
+  if (dtype) GO(float); else GO(bf16_t);
+#undef GO
   VLM_CHECK_LAUNCH();
   return VLM_OK;
 }
 
+extern "C" int vlm_latent_kv_write(const void* d, long ldd, const void* w, int R, int Dr, const void* inv_freq, const void* tok_seq,
+                                   const void* tok_pos, const void* block_table, int max_pages, void* pool, float eps, int rot_half,
+                                   int rows, int dtype, void* stream) {
+  vlm_latent_prep_args a = {};
+  a.d = d; a.ldd = ldd; a.w = w; a.R = R; a.Dr = Dr; a.inv_freq = (const float*)inv_freq; a.amp = 1.f; a.rot_half = rot_half;
+  a.tok_seq = (const int*)tok_seq; a.tok_pos = (const int*)tok_pos; a.block_table = (const int*)block_table; a.max_pages = max_pages;
+  a.pool = pool; a.eps = eps;
+  return vlm_latent_prep_rows(&a, rows, dtype, stream);
+}
+
 extern "C" int vlm_rope_pairs_rows(const void* q, long ldq, long head_stride, int H, int Dr, const void* inv_freq, const void* tok_pos,
-                                   void* out, long ldo, long out_head_stride, int rot_half, int rows, int dtype, void* stream) {
+                                   void* out, long ldo, long out_head_stride, int rot_half, float amp, int rows, int dtype,
+                                   void* stream) {
   if (!q || !tok_pos || !out || H <= 0 || Dr < 0 || (Dr & 1) || (Dr && !inv_freq) || rows < 0) return VLM_ERR_ARG;
   if (rows == 0 || Dr == 0) return VLM_OK;
   hipStream_t st = (hipStream_t)stream;
   const unsigned nb = (unsigned)(((long)rows * H * (Dr / 2) + 255) / 256);
   if (dtype)
     hipLaunchKernelGGL(rope_pairs_rows_kernel<float>, dim3(nb), dim3(256), 0, st, (const float*)q, ldq, head_stride, H, Dr,
-                       (const float*)inv_freq, (const int*)tok_pos, (float*)out, ldo, out_head_stride, rows, rot_half);
+                       (const float*)inv_freq, (const int*)tok_pos, (float*)out, ldo, out_head_stride, rows, rot_half, amp);
   else
     hipLaunchKernelGGL(rope_pairs_rows_kernel<bf16_t>, dim3(nb), dim3(256), 0, st, (const bf16_t*)q, ldq, head_stride, H, Dr,
-                       (const float*)inv_freq, (const int*)tok_pos, (float*)out, ldo, out_head_stride, rows, rot_half);
+                       (const float*)inv_freq, (const int*)tok_pos, (float*)out, ldo, out_head_stride, rows, rot_half, amp);
   VLM_CHECK_LAUNCH();
   return VLM_OK;
 }
 
 extern "C" int vlm_latent_attn(const void* q, const void* pool, const void* tok_seq, const void* tok_pos, const void* block_table,
-                               int max_pages, int H, int R, int Dr, float scale, int window, const void* gate, long ldgate, void* out,
-                               int rows, int dtype, void* stream) {
+                               int max_pages, int H, int R, int Dr, float scale, int window, const void* sink, const void* gate, long ldgate,
+                               void* out, int rows, int dtype, void* stream) {
   if (!q || !pool || !tok_seq || !tok_pos || !block_table || !out || H <= 0 || R <= 0 || Dr < 0 || max_pages <= 0 || rows < 0 ||
       (gate && ldgate < H))
     return VLM_ERR_ARG;
@@ -470,18 +504,18 @@ extern "C" int vlm_latent_attn(const void* q, const void* pool, const void* tok_
     if (dtype)
       hipLaunchKernelGGL(latent_attn_row_vec_kernel<float>, grid, dim3(256), ldsv, st, (const float*)q, (const float*)pool,
                          (const int*)tok_seq, (const int*)tok_pos, (const int*)block_table, max_pages, H, R, Dr, scale, window,
-                         (const float*)gate, ldgate, (float*)out);
+                         (const float*)sink, (const float*)gate, ldgate, (float*)out);
     else
       hipLaunchKernelGGL(latent_attn_row_vec_kernel<bf16_t>, grid, dim3(256), ldsv, st, (const float*)q, (const bf16_t*)pool,
                          (const int*)tok_seq, (const int*)tok_pos, (const int*)block_table, max_pages, H, R, Dr, scale, window,
-                         (const bf16_t*)gate, ldgate, (float*)out);
+                         (const float*)sink, (const bf16_t*)gate, ldgate, (float*)out);
     VLM_CHECK_LAUNCH();
     return VLM_OK;
   }
   const size_t lds = (size_t)(R + Dr + 256 + 8) * sizeof(float);
 #define GO(T, N)                                                                                                                  \
   hipLaunchKernelGGL((latent_attn_kernel<T, N>), grid, dim3(256), lds, st, (const float*)q, (const T*)pool, (const int*)tok_seq,  \
-                     (const int*)tok_pos, (const int*)block_table, max_pages, H, R, Dr, scale, window, (const T*)gate, ldgate, (float*)out)
+                     (const int*)tok_pos, (const int*)block_table, max_pages, H, R, Dr, scale, window, (const float*)sink, (const T*)gate, ldgate, (float*)out)
   const int nacc = (R + 255) / 256;
   if (dtype) {
     if (nacc == 1) GO(float, 1); else if (nacc == 2) GO(float, 2); else GO(float, 4);
@@ -495,7 +529,7 @@ extern "C" int vlm_latent_attn(const void* q, const void* pool, const void* tok_
 
 extern "C" int vlm_latent_attn_blocks(const void* q, const void* pool, const void* qb_start, const void* qb_count, int nblocks,
                                       const void* tok_seq, const void* tok_pos, const void* block_table, int max_pages, int H, int R,
-                                      int Dr, float scale, int window, const void* gate, long ldgate, void* out, int dtype,
+                                      int Dr, float scale, int window, const void* sink, const void* gate, long ldgate, void* out, int dtype,
                                       void* stream) {
   if (!q || !pool || !qb_start || !qb_count || !tok_seq || !tok_pos || !block_table || !out || H <= 0 || R <= 0 || Dr < 0 ||
       max_pages <= 0 || nblocks < 0 || (gate && ldgate < H))
@@ -516,7 +550,7 @@ extern "C" int vlm_latent_attn_blocks(const void* q, const void* pool, const voi
     }                                                                                                                              \
     hipLaunchKernelGGL((latent_attn_block_kernel<T, N>), grid, dim3(256), lds, st, (const float*)q, (const T*)pool,                \
                        (const int*)qb_start, (const int*)qb_count, (const int*)tok_seq, (const int*)tok_pos,                       \
-                       (const int*)block_table, max_pages, H, R, Dr, scale, window, (const T*)gate, ldgate, (float*)out);          \
+                       (const int*)block_table, max_pages, H, R, Dr, scale, window, (const float*)sink, (const T*)gate, ldgate, (float*)out);          \
   } while (0)
   const int nacc = (R + 255) / 256;
   if (dtype) {

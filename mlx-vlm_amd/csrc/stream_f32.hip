@@ -19,6 +19,11 @@
 //                              x[t] += mult * y[t] (+ mult2 * y2[t])                  (y may be NULL: norm only)
 //                              h[t] = x[t] * rsqrt(mean(x[t]^2) + eps) * (w_offset + w)   (w may be NULL: add only; w_offset 1
 //                                                                                      for weights kept as offsets from one)
+//   vlm_sandwich_step        the residual step of a sublayer that is normed before AND after, with the next reader's norm, in one pass:
+//                              r = y[t] (+ bias) (+ pass[t] * src[t])                 (pass: weight of what the sublayer hands on of its input)
+//                              x[t] <- (init ? 0 : x[t]) + mult * r * rsqrt(mean(r^2) + eps) * wy
+//                              h[t] = x[t] * rsqrt(mean(x[t]^2) + eps) * w, or T(x[t]) without w, or nothing without h
+//                            With ids the row y[ids[t]] is read instead of y[t] (a normed embedding lookup with init = 1, mult = 1).
 //   vlm_logit_cap_rows       out[t][j] = cap * tanh(scale * x[t][j] / cap)    (cap = 0: scale * x alone); x and out each fp32 or bf16, may be
 //                                                                                      the same rows
 #include "common.hpp"
@@ -190,6 +195,118 @@ __global__ __launch_bounds__(256) void scaled_add_rms_kernel(float* __restrict__
   for (int d = threadIdx.x; d < D; d += 256) st_f(h + t * ldh + d, xr[d] * r * (w_offset + ld_f(w + d)));
 }
 
+// V consecutive elements (V = 4: one 16- / 8-byte access)
+template <int V> __device__ __forceinline__ void ldv(const float* p, float* f) {
+  if constexpr (V == 4) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+  } else {
+    f[0] = *p;
+  }
+}
+template <int V> __device__ __forceinline__ void ldv(const bf16_t* p, float* f) {
+  if constexpr (V == 4) {
+    const uint2 a = *reinterpret_cast<const uint2*>(p);
+    f[0] = bf_lo(a.x); f[1] = bf_hi(a.x); f[2] = bf_lo(a.y); f[3] = bf_hi(a.y);
+  } else {
+    f[0] = bf2f(*p);
+  }
+}
+template <int V> __device__ __forceinline__ void stv(float* p, const float* f) {
+  if constexpr (V == 4) *reinterpret_cast<float4*>(p) = make_float4(f[0], f[1], f[2], f[3]);
+  else *p = f[0];
+}
+template <int V> __device__ __forceinline__ void stv(bf16_t* p, const float* f) {
+  if constexpr (V == 4) *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf2(f[0], f[1]), pack_bf2(f[2], f[3]));
+  else *p = f2bf(f[0]);
+}
+
+// workgroup = token; a lane owns the columns (256 i + lane) V .. + V and keeps its part of the row in registers
+template <typename T, int V, int NI>
+__global__ __launch_bounds__(256) void sandwich_kernel(vlm_sandwich_args p) {
+  __shared__ float red[4];
+  const long t = blockIdx.x;
+  const int D = p.D;
+  long yr = t;
+  if (p.ids) {
+    const int id = p.ids[t];
+    yr = id < 0 ? 0 : (id >= p.vocab ? p.vocab - 1 : id);
+  }
+  const T* y = (const T*)p.y + yr * p.ldy;
+  const T* src = p.pass ? (const T*)p.src + t * p.ldsrc : nullptr;
+  const float pw = p.pass ? p.pass[t] : 0.f;
+  float* xr = p.x + t * D;
+  float v[NI][V], xv[NI][V];
+  float q = 0.f;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int d = (256 * i + (int)threadIdx.x) * V;
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[i][j] = xv[i][j] = 0.f;
+    if (d < D) {
+      ldv<V>(y + d, v[i]);
+      if (!p.init) ldv<V>(xr + d, xv[i]);
+      if (p.bias) {
+        float b[V];
+        ldv<V>((const T*)p.bias + d, b);
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[i][j] += b[j];
+      }
+      if (src) {
+        float b[V];
+        ldv<V>(src + d, b);
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[i][j] = fmaf(pw, b[j], v[i][j]);
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) q = fmaf(v[i][j], v[i][j], q);
+    }
+  }
+  const float r = p.mult / sqrtf(block_sum(q, red) / (float)D + p.eps);
+  q = 0.f;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int d = (256 * i + (int)threadIdx.x) * V;
+    if (d < D) {
+      float w[V];
+      ldv<V>((const T*)p.wy + d, w);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        xv[i][j] = fmaf(v[i][j] * r, w[j], xv[i][j]);
+        q = fmaf(xv[i][j], xv[i][j], q);
+      }
+      stv<V>(xr + d, xv[i]);
+    }
+  }
+  if (!p.h) return;
+  const float r2 = p.w ? 1.0f / sqrtf(block_sum(q, red) / (float)D + p.eps) : 1.f;
+  T* h = (T*)p.h + t * p.ldh;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int d = (256 * i + (int)threadIdx.x) * V;
+    if (d < D) {
+      if (p.w) {
+        float w[V];
+        ldv<V>((const T*)p.w + d, w);
+#pragma unroll
+        for (int j = 0; j < V; ++j) xv[i][j] *= r2 * w[j];
+      }
+      stv<V>(h + d, xv[i]);
+    }
+  }
+}
+
+template <typename T, int V>
+int sandwich_launch(const vlm_sandwich_args& a, int rows, hipStream_t st) {
+  const int n = (a.D + 256 * V - 1) / (256 * V);
+#define GO(N) hipLaunchKernelGGL((sandwich_kernel<T, V, N>), dim3(rows), dim3(256), 0, st, a)
+  if (n <= 1) GO(1); else if (n <= 2) GO(2); else if (n <= 4) GO(4); else if (n <= 8) GO(8); else if (n <= 16) GO(16); else if (n <= 32) GO(32);
+  else return VLM_ERR_SHAPE;
+#undef GO
+  VLM_CHECK_LAUNCH();
+  return VLM_OK;
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void relu2_rows_kernel(const T* __restrict__ in, long ldi, T* __restrict__ out, long ldo, int rows,
                                                          int dim) {
@@ -333,6 +450,20 @@ extern "C" int vlm_scaled_add_rms(void* x, const void* y, long ldy, float mult, 
   else hipLaunchKernelGGL((scaled_add_rms_kernel<bf16_t, bf16_t>), dim3(rows), dim3(256), 0, st, (float*)x, (const bf16_t*)y, ldy, mult, (const bf16_t*)y2, ldy2, mult2, (const bf16_t*)w, w_offset, (bf16_t*)h, ldh, D, eps);
   VLM_CHECK_LAUNCH();
   return VLM_OK;
+}
+
+extern "C" int vlm_sandwich_step(const vlm_sandwich_args* a, int rows, int dtype, void* stream) {
+  if (!a || !a->x || !a->y || !a->wy || !STREAM_ARGS_OK(rows, a->D) || a->ldy < a->D || (a->ids && a->vocab <= 0) ||
+      (a->pass && (!a->src || a->ldsrc < a->D)) || (a->h && a->ldh < a->D) || (a->w && !a->h))
+    return VLM_ERR_ARG;
+  if (rows == 0) return VLM_OK;
+  hipStream_t st = (hipStream_t)stream;
+  const size_t es = dtype ? 4 : 2;
+  const uintptr_t ptrs = (uintptr_t)a->y | (uintptr_t)a->bias | (uintptr_t)a->src | (uintptr_t)a->wy | (uintptr_t)a->w | (uintptr_t)a->h;
+  const bool vec = a->D % 4 == 0 && a->ldy % 4 == 0 && (!a->pass || a->ldsrc % 4 == 0) && (!a->h || a->ldh % 4 == 0) &&
+                   ptrs % (4 * es) == 0 && (uintptr_t)a->x % 16 == 0;
+  if (dtype) return vec ? sandwich_launch<float, 4>(*a, rows, st) : sandwich_launch<float, 1>(*a, rows, st);
+  return vec ? sandwich_launch<bf16_t, 4>(*a, rows, st) : sandwich_launch<bf16_t, 1>(*a, rows, st);
 }
 
 extern "C" int vlm_logit_cap_rows(const void* x, long ldx, int x_f32, void* out, long ldo, int out_f32, int rows, int dim, float scale, float cap,

@@ -4,11 +4,10 @@ lives in the model code and the kernels.  Unknown mixer types / feed-forward kin
 from __future__ import annotations
 
 import copy
-import math
 from dataclasses import dataclass, field
 from typing import Any, Dict, List, Optional
 
-import numpy as np
+from ..ragged import rotation  # noqa: F401   (the frequency table of a `rot` entry)
 
 MIXERS = ("lightning", "attention")
 MAX_STREAMS, MAX_TAPS, MAX_VDIM = 8, 16, 256          # what the kernels take
@@ -18,29 +17,6 @@ def _need(d: Dict[str, Any], keys, what: str):
     missing = [k for k in keys if k not in d]
     if missing:
         raise ValueError(f"Zivitar {what}: missing {missing}")
-
-
-def rotation(rot: Optional[Dict[str, Any]]):
-    """-> (rotated dimensions, fp32 frequency per pair (numpy), factor on cos and sin).  Plain frequencies are base^(-2 i / dims).
-    With `scaling`, a pair that turns fewer than `slow` times over `original` positions has its frequency divided by `factor`, one that
-    turns more than `fast` times keeps it, a linear ramp over the pair index lies between, and cos and sin grow by 0.1 ln(factor) + 1."""
-    if not rot or not int(rot.get("dims", 0)):
-        return 0, None, 1.0
-    dims, base = int(rot["dims"]), float(rot["base"])
-    i = np.arange(dims // 2, dtype=np.float64)
-    f = base ** (-2.0 * i / dims)
-    sc = rot.get("scaling")
-    if not sc:
-        return dims, f.astype(np.float32), 1.0
-    factor = float(sc["factor"])
-
-    def pair(turns: float) -> float:          # the pair index that turns `turns` times over `original` positions
-        return dims * math.log(float(sc["original"]) / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
-
-    lo = max(math.floor(pair(float(sc["fast"]))), 0)
-    hi = min(math.ceil(pair(float(sc["slow"]))), dims - 1)
-    ramp = np.clip((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
-    return dims, (f / factor * ramp + f * (1.0 - ramp)).astype(np.float32), 0.1 * math.log(factor) + 1.0
 
 
 @dataclass

@@ -651,38 +651,66 @@ def latent_kv_write(d, w, R, Dr, inv_freq, tok_seq, tok_pos, block_table, pool, 
                                          _f32(d), _stream()), "latent_kv_write")
 
 
-def rope_pairs_rows(q, head_stride, H, Dr, inv_freq, tok_pos, out, out_head_stride, rot_half=False):
-    """rotation of a Dr-wide part of every head (pairs (2 i, 2 i + 1), or (i, i + Dr / 2) with rot_half): q / out are 2-D views
-    at the part's first column"""
+def latent_prep_rows(d, w, R, Dr, inv_freq, tok_seq, tok_pos, block_table, pool, eps, amp=1.0, rot_half=False, dq=None, wq=None, cq=None):
+    """latent_kv_write with a factor on cos and sin; dq (2-D view [T, Rq]) / wq [Rq]: the query's own latent, RMS-normed into cq in the same
+    launch (returned)"""
+    _dev(d, w, inv_freq, tok_seq, tok_pos, block_table, pool, dq, wq, cq)
+    a = _lib.LatentPrepArgs()
+    a.d, a.ldd, a.w, a.R, a.Dr, a.inv_freq, a.amp, a.rot_half = _p(d), d.stride(0), _p(w), int(R), int(Dr), _p(inv_freq), float(amp), int(bool(rot_half))
+    a.tok_seq, a.tok_pos, a.block_table, a.max_pages = _p(tok_seq), _p(tok_pos), _p(block_table), block_table.shape[1]
+    a.pool, a.eps = _p(pool), float(eps)
+    if pool.dtype != d.dtype or pool.shape[-1] != R + Dr:
+        raise _lib.VlmHipError("latent_prep_rows: a pool of rows [R + Dr] in the rows' dtype expected")
+    if dq is not None:
+        Rq = wq.numel()
+        if cq is None:
+            cq = torch.empty(d.shape[0], (Rq + 7) & ~7, dtype=d.dtype, device=d.device)[:, :Rq]
+        if dq.dtype != d.dtype or wq.dtype != d.dtype or cq.dtype != d.dtype:
+            raise _lib.VlmHipError("latent_prep_rows: one dtype for both latents expected")
+        a.dq, a.lddq, a.wq, a.Rq, a.cq, a.ldcq = _p(dq), dq.stride(0), _p(wq), Rq, _p(cq), cq.stride(0)
+    check(_lib.lib().vlm_latent_prep_rows(C.byref(a), d.shape[0], _f32(d), _stream()), "latent_prep_rows")
+    return cq
+
+
+def rope_pairs_rows(q, head_stride, H, Dr, inv_freq, tok_pos, out, out_head_stride, rot_half=False, amp=1.0):
+    """rotation of a Dr-wide part of every head (pairs (2 i, 2 i + 1), or (i, i + Dr / 2) with rot_half; cos and sin times amp): q / out
+    are 2-D views at the part's first column"""
     _dev(q, inv_freq, tok_pos, out)
     check(_lib.lib().vlm_rope_pairs_rows(_p(q), q.stride(0), int(head_stride), int(H), int(Dr), _p(inv_freq), _p(tok_pos), _p(out),
-                                         out.stride(0), int(out_head_stride), int(bool(rot_half)), q.shape[0], _f32(q), _stream()),
+                                         out.stride(0), int(out_head_stride), int(bool(rot_half)), float(amp), q.shape[0], _f32(q), _stream()),
           "rope_pairs_rows")
 
 
-def latent_attn(q, pool, tok_seq, tok_pos, block_table, H, R, Dr, scale, gate=None, out=None, window=0):
+def _sink_ok(sink, H):
+    if sink is not None and (sink.dtype != torch.float32 or sink.numel() != H or not sink.is_contiguous()):
+        raise _lib.VlmHipError("attention: fp32 sinks, one per head, expected")
+
+
+def latent_attn(q, pool, tok_seq, tok_pos, block_table, H, R, Dr, scale, gate=None, out=None, window=0, sink=None):
     """q fp32 [T, H, R + Dr] over the latent pool -> fp32 [T, H, R] (times sigmoid(gate[t, h]) when given); window > 0: a query
-    reaches back window - 1 tokens"""
-    _dev(q, pool, tok_seq, tok_pos, block_table, gate, out)
+    reaches back window - 1 tokens; sink fp32 [H]: exp(sink[h]) in the softmax's denominator"""
+    _dev(q, pool, tok_seq, tok_pos, block_table, gate, out, sink)
+    _sink_ok(sink, H)
     T = q.shape[0]
     if out is None:
         out = torch.empty(T, H, R, dtype=torch.float32, device=q.device)
     check(_lib.lib().vlm_latent_attn(_p(q), _p(pool), _p(tok_seq), _p(tok_pos), _p(block_table), block_table.shape[1], int(H), int(R),
-                                     int(Dr), float(scale), int(window), _p(gate), gate.stride(0) if gate is not None else 0, _p(out), T,
-                                     _f32(pool), _stream()), "latent_attn")
+                                     int(Dr), float(scale), int(window), _p(sink), _p(gate), gate.stride(0) if gate is not None else 0,
+                                     _p(out), T, _f32(pool), _stream()), "latent_attn")
     return out
 
 
-def latent_attn_blocks(q, pool, qb_start, qb_count, tok_seq, tok_pos, block_table, H, R, Dr, scale, gate=None, out=None, window=0):
+def latent_attn_blocks(q, pool, qb_start, qb_count, tok_seq, tok_pos, block_table, H, R, Dr, scale, gate=None, out=None, window=0, sink=None):
     """latent_attn over query blocks (qb_start / qb_count int32 [n]: first token and number of consecutive tokens of one
     sequence, at most 16): the prompt form, key tiles staged once per block"""
-    _dev(q, pool, qb_start, qb_count, tok_seq, tok_pos, block_table, gate, out)
+    _dev(q, pool, qb_start, qb_count, tok_seq, tok_pos, block_table, gate, out, sink)
+    _sink_ok(sink, H)
     T = q.shape[0]
     if out is None:
         out = torch.empty(T, H, R, dtype=torch.float32, device=q.device)
     check(_lib.lib().vlm_latent_attn_blocks(_p(q), _p(pool), _p(qb_start), _p(qb_count), qb_start.numel(), _p(tok_seq), _p(tok_pos),
                                             _p(block_table), block_table.shape[1], int(H), int(R), int(Dr), float(scale), int(window),
-                                            _p(gate), gate.stride(0) if gate is not None else 0, _p(out), _f32(pool), _stream()),
+                                            _p(sink), _p(gate), gate.stride(0) if gate is not None else 0, _p(out), _f32(pool), _stream()),
           "latent_attn_blocks")
     return out
 
@@ -711,20 +739,61 @@ def moe_route_scored(logits, top, groups=1, keep=1, scale=1.0):
     return gate, idx, wgt
 
 
-GLU_GELU_TANH, GLU_SILU, GLU_SIGMOID, GLU_CLAMPED = 0, 1, 2, 3
+GLU_GELU_TANH, GLU_SILU, GLU_SIGMOID, GLU_CLAMPED, GLU_RELU = 0, 1, 2, 3, 4
 
 
-def glu_rows(g, u, act, out=None, route=None, E=0, ff=0, estride=0, limit=float("inf")):
-    """out = act(g) * u (GLU_CLAMPED: g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' within +-limit) over 2-D views with a row pitch (dim: out's columns, else g's); with route (fp32 [T, E]): out [T, E * ff], expert e reads the
-    columns e * estride .. + ff of g and u, times route[t, e]"""
-    _dev(g, u, out, route)
+def glu_rows(g, u, act, out=None, route=None, E=0, ff=0, estride=0, limit=float("inf"), gbias=None, ubias=None):
+    """out = act(g) * u (GLU_CLAMPED: g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' within +-limit) over 2-D views with a row
+    pitch (dim: out's columns, else g's); with route (fp32 [T, E]): out [T, E * ff], expert e reads the columns e * estride .. + ff of
+    g and u, times route[t, e]; gbias / ubias [dim]: added to g and u first (without route)"""
+    _dev(g, u, out, route, gbias, ubias)
     rows = g.shape[0]
     dim = int(E) * int(ff) if route is not None else (out.shape[1] if out is not None else g.shape[1])
     if out is None:
         out = torch.empty(rows, dim, dtype=g.dtype, device=g.device)
+    for b in (gbias, ubias):
+        if b is not None and (b.dtype != g.dtype or b.numel() != dim):
+            raise _lib.VlmHipError("glu_rows: biases have one entry per output column, in the rows' dtype")
     check(_lib.lib().vlm_glu_rows(_p(g), g.stride(0), _p(u), u.stride(0), _p(route), int(E), int(ff), int(estride or ff), int(act), float(limit),
-                                  _p(out), out.stride(0), rows, dim, _f32(g), _stream()), "glu_rows")
+                                  _p(gbias), _p(ubias), _p(out), out.stride(0), rows, dim, _f32(g), _stream()), "glu_rows")
     return out
+
+
+def moe_router_softmax(h, w, top, identity=0, correction=None):
+    """rows h [T, D], router w [E, D] -> (gate table fp32 [T, E - identity], identity weights fp32 [T] or None): softmax scores over all E
+    columns, the `top` largest of score + correction keep their score; the last `identity` columns hand their input on"""
+    _dev(h, w, correction)
+    T, D = h.shape
+    E = w.shape[0]
+    if w.dtype != h.dtype or w.shape[1] != D or (correction is not None and (correction.dtype != torch.float32 or correction.numel() != E)):
+        raise _lib.VlmHipError("moe_router_softmax: router rows of h's width and dtype, fp32 correction per column expected")
+    gate = torch.empty(T, E - identity, dtype=torch.float32, device=h.device)
+    ident = torch.empty(T, dtype=torch.float32, device=h.device) if identity else None
+    check(_lib.lib().vlm_moe_router_softmax(_p(h), h.stride(0), _p(w), w.stride(0), D, T, E, int(top), int(identity), _p(correction),
+                                            _p(gate) if identity < E else None, _p(ident), _f32(h), _stream()), "moe_router_softmax")
+    return gate, ident
+
+
+def sandwich_step(x, y, wy, mult=1.0, w=None, eps=1e-6, bias=None, pass_=None, src=None, ids=None, init=False, h=None, cast=False):
+    """r = y (+ bias) (+ pass_[t] * src[t]);  x <- (0 if init else x) + mult * rms(r) * wy;  returns h = rms(x) * w (or, with cast, x itself
+    in wy's dtype; None with neither).  ids: row ids[t] of the table y instead of row t.  x: contiguous fp32 [T, D], in place."""
+    _dev(x, y, wy, w, bias, pass_, src, ids, h)
+    T, D = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous() or y.dtype != wy.dtype or y.shape[1] < D or wy.numel() != D:
+        raise _lib.VlmHipError("sandwich_step: contiguous fp32 stream, rows of its width in wy's dtype expected")
+    if (ids is None and y.shape[0] != T) or (ids is not None and (ids.dtype != torch.int32 or ids.numel() != T)):
+        raise _lib.VlmHipError("sandwich_step: one row (or one int32 id) per stream row expected")
+    if pass_ is not None and (pass_.dtype != torch.float32 or pass_.numel() != T or src is None or src.dtype != y.dtype or src.shape[0] != T):
+        raise _lib.VlmHipError("sandwich_step: fp32 pass weight per row and source rows expected")
+    if h is None and (w is not None or cast):
+        h = torch.empty(T, D, dtype=wy.dtype, device=x.device)
+    a = _lib.SandwichArgs()
+    a.x, a.init, a.ids, a.vocab, a.y, a.ldy, a.bias = _p(x), int(bool(init)), _p(ids), y.shape[0], _p(y), y.stride(0), _p(bias)
+    if pass_ is not None:
+        a.pass_, a.src, a.ldsrc = _p(pass_), _p(src), src.stride(0)
+    a.wy, a.mult, a.w, a.h, a.ldh, a.D, a.eps = _p(wy), float(mult), _p(w), _p(h), h.stride(0) if h is not None else 0, D, float(eps)
+    check(_lib.lib().vlm_sandwich_step(C.byref(a), T, _f32(wy), _stream()), "sandwich_step")
+    return h
 
 
 def scaled_add_rms_(x, y=None, mult=1.0, w=None, w_offset=0.0, eps=1e-6, h=None, y2=None, mult2=1.0, h_dtype=None):
@@ -1034,6 +1103,76 @@ def diff_attn_rows(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv,
     a = _diff_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, lam, mult, eps, out, window, keep)
     a.nsplit, a.part = nsplit, _p(part)
     check(_lib.lib().vlm_diff_attn_rows(C.byref(a), tok_seq.numel(), _f32(vpool), _stream()), "diff_attn_rows")
+    return out
+
+
+def qkv_rownorm_rows(x, offs, HQ, HK, D, NV, qw, kw, eps, tok_seq, tok_pos, block_table, q, kpool, vpool, qbias=None, kbias=None, vbias=None,
+                     temp=None, vother=None, mix=0.0):
+    """Packed projection rows x (parts at columns offs = (q, k, v)) + biases -> q fp32 [T, HQ * D] and k into its paged pool, each RMS-normed
+    over all heads at once times a weight (q also times 1 + coef * ln(floor((pos + 1) / every) + 1) with temp = (coef, every)); v into its
+    pool, mixed with the token's row of another value pool: (1 - mix) v + mix vother.  Key pool: fp32 rows [HK * D], or bf16 rows
+    diff_key_width(HK, D) (every coordinate as two bf16 values)."""
+    _dev(x, qw, kw, tok_seq, tok_pos, block_table, q, kpool, vpool, qbias, kbias, vbias, vother)
+    T = x.shape[0]
+    split = kpool.dtype == torch.bfloat16
+    if q.dtype != torch.float32 or q.numel() != T * HQ * D or kpool.shape[-1] != diff_key_width(HK, D, split) or vpool.shape[-1] != NV:
+        raise _lib.VlmHipError("qkv_rownorm_rows: fp32 q rows [T, HQ * D], a key pool of HK heads, value pool [.., NV] expected")
+    if any(b is not None and b.dtype != x.dtype for b in (qw, kw, qbias, kbias, vbias, vpool, vother)) or qw.numel() != HQ * D or kw.numel() != HK * D \
+            or (vother is not None and vother.shape != vpool.shape):
+        raise _lib.VlmHipError("qkv_rownorm_rows: weights, biases and value pools of the rows' dtype, one weight per coordinate expected")
+    a = _lib.QkvRownormArgs()
+    a.x, a.ldx, (a.qoff, a.koff, a.voff) = _p(x), x.stride(0), (int(o) for o in offs)
+    a.HQ, a.HK, a.D, a.NV, a.eps = int(HQ), int(HK), int(D), int(NV), float(eps)
+    a.qbias, a.kbias, a.vbias, a.qw, a.kw = _p(qbias), _p(kbias), _p(vbias), _p(qw), _p(kw)
+    if temp is not None:
+        a.temp_coef, a.temp_every = float(temp[0]), int(temp[1])
+    a.tok_seq, a.tok_pos, a.block_table, a.max_pages = _p(tok_seq), _p(tok_pos), _p(block_table), block_table.shape[1]
+    a.q, a.kpool, a.vpool, a.vother, a.mix, a.k_split = _p(q), _p(kpool), _p(vpool), _p(vother), float(mix), int(split)
+    check(_lib.lib().vlm_qkv_rownorm_rows(C.byref(a), T, _f32(x), _stream()), "qkv_rownorm_rows")
+    return q
+
+
+def _grouped_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, out, window, slope, sink, gate):
+    if q.dtype != torch.float32 or kpool.dtype != vpool.dtype or vpool.dtype != out.dtype or not q.is_contiguous():
+        raise _lib.VlmHipError("grouped_attn: fp32 queries; keys, values and output of one dtype expected")
+    if kpool.shape[-1] != diff_key_width(KH, D, kpool.dtype == torch.bfloat16) or vpool.shape[-1] != KH * Dv or q.numel() != tok_seq.numel() * H * D:
+        raise _lib.VlmHipError("grouped_attn: D key coordinates and Dv value columns per head expected")
+    _sink_ok(sink, H)
+    _sink_ok(slope, H)
+    if gate is not None and gate.dtype != out.dtype:
+        raise _lib.VlmHipError("grouped_attn: the gate has the output's dtype")
+    a = _lib.GroupedAttnArgs()
+    a.q, a.kpool, a.vpool, a.tok_seq, a.tok_pos, a.block_table = _p(q), _p(kpool), _p(vpool), _p(tok_seq), _p(tok_pos), _p(block_table)
+    a.max_pages, a.H, a.KH, a.D, a.Dv, a.scale, a.window = block_table.shape[1], int(H), int(KH), int(D), int(Dv), float(scale), int(window)
+    a.slope, a.sink, a.gate, a.ldgate, a.out, a.ldo = _p(slope), _p(sink), _p(gate), gate.stride(0) if gate is not None else 0, _p(out), out.stride(0)
+    return a
+
+
+def grouped_attn_blocks(q, kpool, vpool, qb_start, qb_count, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, out, window=0, slope=None,
+                        sink=None, gate=None):
+    """grouped-head softmax attention, prompt form: q fp32 [T, H * D], pools with rows [diff_key_width(KH, D)] / [KH * Dv] in the serving
+    dtype, out [T, H * Dv].  Scores (q . k) scale - slope[h] (i - j) inside the window; exp(sink[h]) in the denominator; read-outs times
+    sigmoid(gate[t, h])"""
+    _dev(q, kpool, vpool, qb_start, qb_count, tok_seq, tok_pos, block_table, out, slope, sink, gate)
+    a = _grouped_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, out, window, slope, sink, gate)
+    a.qb_start, a.qb_count = _p(qb_start), _p(qb_count)
+    check(_lib.lib().vlm_grouped_attn_blocks(C.byref(a), qb_start.numel(), _f32(vpool), _stream()), "grouped_attn_blocks")
+    return out
+
+
+def grouped_attn_rows(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, out, window=0, slope=None, sink=None, gate=None,
+                      nsplit=None):
+    """grouped-head softmax attention, decode form: one token and the heads that share a key / value head per workgroup; few such column
+    groups share their keys between several workgroups each (merged by a second kernel)"""
+    _dev(q, kpool, vpool, tok_seq, tok_pos, block_table, out, slope, sink, gate)
+    rows = tok_seq.numel()
+    groups = rows * KH * -(-(H // KH) // 16)
+    span = min(block_table.shape[1] * 64, window if window > 0 else 1 << 30)             # keys a query can see
+    nsplit = max(1, min(256 // max(groups, 1), -(-span // 128), 32)) if nsplit is None else int(nsplit)
+    part = torch.empty(nsplit, H, rows, Dv + 2, dtype=torch.float32, device=q.device) if nsplit > 1 else None
+    a = _grouped_attn_args(q, kpool, vpool, tok_seq, tok_pos, block_table, H, KH, D, Dv, scale, out, window, slope, sink, gate)
+    a.nsplit, a.part = nsplit, _p(part)
+    check(_lib.lib().vlm_grouped_attn_rows(C.byref(a), rows, _f32(vpool), _stream()), "grouped_attn_rows")
     return out
 
 
