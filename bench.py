@@ -107,7 +107,7 @@ def main():
                     help="336x336 images per vision-tower call of the ViT throughput line (16 = the workload of rounds 1-4 is reported "
                          "next to it; 68 images, where every GEMM fills its last round of 256 workgroups, measured +0.4 %: the tail of a "
                          "launch is not a whole round)")
-    ap.add_argument("--workload", default="qwen2vl-2b", choices=["qwen2vl-2b", "nanollava", "qwen2vl-7b-b32", "qwen2vl-2b-w4", "phi35v-w4-b16", "idefics2-b8", "garesun-compare", "luvapel-compare", "tilalorn-compare", "dimudra-compare", "zivitar-compare"])
+    ap.add_argument("--workload", default="qwen2vl-2b", choices=["qwen2vl-2b", "nanollava", "qwen2vl-7b-b32", "qwen2vl-2b-w4", "phi35v-w4-b16", "idefics2-b8", "garesun-compare", "luvapel-compare", "tilalorn-compare", "dimudra-compare", "zivitar-compare", "rorovik-compare"])
     ap.add_argument("--kv-bits", type=int, default=0, help="phi35v-w4-b16: 8 = uniform 8-bit KV cache (kv_bits of the reference)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-cpu-hf", action="store_true", help="skip the HuggingFace torch-CPU second opinion of cpu_baseline")
@@ -176,6 +176,11 @@ def main():
         # likewise: the Zivitar design next to Luvapel (recurrences, windowed attention and dense feed-forwards on the same ragged step)
         from benchlib.zivitar import workload_zivitar_compare
         print(json.dumps(workload_zivitar_compare(args)), flush=True)
+        return
+    if args.workload == "rorovik-compare":
+        # likewise: the Rorovik design next to Tilalorn (latent and grouped attention, dense and expert feed-forwards on the same ragged step)
+        from benchlib.rorovik import workload_rorovik_compare
+        print(json.dumps(workload_rorovik_compare(args)), flush=True)
         return
     if args.workload != "qwen2vl-2b":
         rank, ws, local = parallel.init()

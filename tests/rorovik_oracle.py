@@ -74,8 +74,8 @@ def sink_softmax(scores, vis, sink):
 
 
 def temperature(T, qt, dtype):
-    p = torch.arange(T)
-    return 1.0 + qt["coef"] * torch.log(torch.floor((p + 1) / qt["every"]) + 1.0).to(dtype)
+    steps = (torch.arange(T) + 1) // qt["every"]
+    return 1.0 + qt["coef"] * torch.log(steps.to(dtype) + 1.0)
 
 
 def slopes(H, dtype):
