@@ -626,8 +626,8 @@ int vlm_latent_kv_write(const void* d, long ldd, const void* w, int R, int Dr, c
                         int dtype, void* stream);
 /* rot_half (both functions above and below): 0 = the rotated pairs are (2 i, 2 i + 1), 1 = (i, i + Dr / 2).  ABI v11. */
 int vlm_rope_pairs_rows(const void* q, long ldq, long head_stride, int H, int Dr, const void* inv_freq, const void* tok_pos, void* out,
-                        long ldo, long out_head_stride, int rot_half, float amp, int rows, int dtype, void* stream);
-/* ABI v14: amp: a factor on cos and sin (above and below); vlm_latent_kv_write with it, and with dq the RMS norm of the query's own latent
+                        long ldo, long out_head_stride, int rot_half, float amp, int out_f32, int rows, int dtype, void* stream);
+/* ABI v14: amp: a factor on cos and sin (above and below); out_f32: fp32 output rows, else T; vlm_latent_kv_write with it, and with dq the RMS norm of the query's own latent
  * (T rows [Rq] at lddq -> cq) in the same launch. */
 typedef struct vlm_latent_prep_args {
   const void* d;                        /* T rows [R + Dr] at ldd */
@@ -659,6 +659,27 @@ int vlm_latent_attn(const void* q, const void* pool, const void* tok_seq, const 
 int vlm_latent_attn_blocks(const void* q, const void* pool, const void* qb_start, const void* qb_count, int nblocks, const void* tok_seq,
                            const void* tok_pos, const void* block_table, int max_pages, int H, int R, int Dr, float scale, int window,
                            const void* sink, const void* gate, long ldgate, void* out, int dtype, void* stream);
+
+/* csrc/latent_attn_mfma.hip (ABI v14): the same attention on the bf16 matrix cores over bf16 pools, R % 8 == 0, Dr % 8 == 0, R <= 512,
+ * R + Dr <= 576, 16-byte aligned pointers: _blocks for query blocks (prompt form), _rows for single tokens (nsplit workgroups share a
+ * token's keys). */
+typedef struct vlm_latent_mfma_args {
+  const void* q;                        /* bf16 [tokens][H][R + Dr] */
+  const void* pool;                     /* bf16 [pages][64][R + Dr] */
+  const int *qb_start, *qb_count;       /* _blocks only */
+  const int *tok_seq, *tok_pos, *block_table;
+  int max_pages, H, R, Dr;
+  float scale;
+  int window;                           /* <= 0: every earlier key */
+  const float* sink;                    /* fp32 [H] or NULL */
+  const void* gate;                     /* bf16 rows [H] at ldgate or NULL */
+  long ldgate;
+  void* out;                            /* bf16 [tokens][H][R] */
+  int nsplit;                           /* _rows: 0 / 1: one workgroup per token and 16 heads; at most 64 */
+  float* part;                          /* nsplit > 1: scratch fp32 [nsplit][H][rows][R + 2] */
+} vlm_latent_mfma_args;
+int vlm_latent_attn_mfma_blocks(const vlm_latent_mfma_args* a, int nblocks, void* stream);
+int vlm_latent_attn_mfma_rows(const vlm_latent_mfma_args* a, int rows, void* stream);
 
 /* csrc/moe.hip */
 int vlm_moe_route(const void* logits, int T, int E, int top, void* gate, void* idx, void* wgt, void* stream);

@@ -166,6 +166,13 @@ class LatentPrepArgs(C.Structure):
                 ("ldcq", C.c_long)]
 
 
+class LatentMfmaArgs(C.Structure):
+    """vlm_latent_mfma_args (include/vlm_hip.h)"""
+    _fields_ = ([(n, c_void_p) for n in ("q", "pool", "qb_start", "qb_count", "tok_seq", "tok_pos", "block_table")]
+                + [(n, c_int) for n in ("max_pages", "H", "R", "Dr")] + [("scale", c_float), ("window", c_int), ("sink", c_void_p), ("gate", c_void_p),
+                                                                         ("ldgate", C.c_long), ("out", c_void_p), ("nsplit", c_int), ("part", c_void_p)])
+
+
 class SandwichArgs(C.Structure):
     """vlm_sandwich_args (include/vlm_hip.h)"""
     _fields_ = [("x", c_void_p), ("init", c_int), ("ids", c_void_p), ("vocab", c_int), ("y", c_void_p), ("ldy", C.c_long), ("bias", c_void_p),
@@ -297,11 +304,13 @@ SIGNATURES = {
     "vlm_latent_kv_write": (c_int, [c_void_p, C.c_long, c_void_p, c_int, c_int] + [c_void_p] * 4 + [c_int, c_void_p, c_float, c_int,
                                     c_int, c_int, c_void_p]),
     "vlm_rope_pairs_rows": (c_int, [c_void_p, C.c_long, C.c_long, c_int, c_int, c_void_p, c_void_p, c_void_p, C.c_long, C.c_long,
-                                    c_int, c_float, c_int, c_int, c_void_p]),
+                                    c_int, c_float, c_int, c_int, c_int, c_void_p]),
     "vlm_latent_prep_rows": (c_int, [P(LatentPrepArgs), c_int, c_int, c_void_p]),
     "vlm_latent_attn": (c_int, [c_void_p] * 5 + [c_int] * 4 + [c_float, c_int, c_void_p, c_void_p, C.c_long, c_void_p, c_int, c_int, c_void_p]),
     "vlm_latent_attn_blocks": (c_int, [c_void_p] * 4 + [c_int] + [c_void_p] * 3 + [c_int] * 4 + [c_float, c_int, c_void_p, c_void_p, C.c_long,
                                        c_void_p, c_int, c_void_p]),
+    "vlm_latent_attn_mfma_blocks": (c_int, [P(LatentMfmaArgs), c_int, c_void_p]),
+    "vlm_latent_attn_mfma_rows": (c_int, [P(LatentMfmaArgs), c_int, c_void_p]),
     "vlm_sandwich_step": (c_int, [P(SandwichArgs), c_int, c_int, c_void_p]),
     "vlm_qkv_rownorm_rows": (c_int, [P(QkvRownormArgs), c_int, c_int, c_void_p]),
     "vlm_grouped_attn_blocks": (c_int, [P(GroupedAttnArgs), c_int, c_int, c_void_p]),

@@ -175,6 +175,18 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
   }
   const int* bt = p.block_table + (long)p.tok_seq[t0] * p.max_pages;
   const int pos0 = p.tok_pos[t0], last = decode ? pos0 : pos0 + ncol - 1;
+  const int window = p.window;
+  const int tiles = last / KTL + 1;
+  const int first_tile = window > 0 ? max(0, pos0 - window + 1) / KTL : 0;   // holds the first query's oldest visible key
+  const bool split = gridDim.z > 1;
+  if (split && first_tile + (int)blockIdx.z * NW >= tiles) {              // no keys for this workgroup: only the marks of an empty part (uniform)
+    if (tid < ncol) {
+      float* q = p.part + (((long)blockIdx.z * p.H + h0 + tid) * gridDim.x + t0) * (Dv + 2);
+      q[Dv] = -INFINITY;
+      q[Dv + 1] = 0.f;
+    }
+    return;
+  }
   const float sc = p.scale * LOG2E;
   const int dq = F32 ? DP : DPB;
   for (int i = tid; i < CG * QC * dq; i += NW * 64) {
@@ -195,7 +207,6 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
   }
   __syncthreads();
   const int mypos = r16 < ncol ? (decode ? pos0 : pos0 + r16) : -1;       // (a column that does not exist sees nothing)
-  const int window = p.window;
   float slope[CG];                                       // of this lane's column, times log2(e)
 #pragma unroll
   for (int m = 0; m < CG; ++m) slope[m] = p.slope ? p.slope[decode ? h0 + min(r16, ncol - 1) : h0 + m] * LOG2E : 0.f;
@@ -210,8 +221,6 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
     mrun[m] = -INFINITY;
     lrun[m] = 0.f;
   }
-  const int tiles = last / KTL + 1;
-  const int first_tile = window > 0 ? max(0, pos0 - window + 1) / KTL : 0;   // holds the first query's oldest visible key
   const bool dvec = (D & 3) == 0, vvec = Dv % NB == 0;
   const int vcol = r16 * NB, vhave = Dv - vcol;
   const long krow_sz = F32 ? (long)p.KH * D : (long)p.KH * 2 * D8, vrow_sz = (long)p.KH * Dv;
@@ -308,7 +317,6 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
     }
   }
   __syncthreads();
-  const bool split = gridDim.z > 1;
 #pragma unroll
   for (int m = 0; m < CG; ++m) {
     float M = -INFINITY;
@@ -357,7 +365,7 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
 }
 
 // merge of the splits' partial results: grid (rows, H), 2 waves (wave w: every other 64 value columns from 64 w).
-// part: [split][H][rows][Dv sums | maximum | sum]
+// part: [split][H][rows][Dv sums | maximum | sum]; the splits that had keys come first
 template <typename T>
 __global__ __launch_bounds__(128) void grouped_attn_merge_kernel(vlm_grouped_attn_args p, int nsplit) {
   const long t = blockIdx.x;
@@ -370,15 +378,16 @@ __global__ __launch_bounds__(128) void grouped_attn_merge_kernel(vlm_grouped_att
   float l = wave_sum(l_mine * f_mine);
   if (p.sink) l += __builtin_amdgcn_exp2f(p.sink[h] * LOG2E - ms);
   const float inv = (l > 0.f ? 1.f / l : 0.f) * head_gate<T>(p, t, h);
+  const int n = __popcll(__ballot(M_mine != -INFINITY));
   for (int c0 = 64 * wave; c0 < Dv; c0 += 128) {         // (whole waves: the shuffles below need every lane)
     const int c = min(c0 + lane, Dv - 1);
     float a = 0.f;
-    for (int z0 = 0; z0 < nsplit; z0 += 8) {             // eight loads in flight; splits past the last one count for nothing
+    for (int z0 = 0; z0 < n; z0 += 8) {             // eight loads in flight; splits past the last one count for nothing
       float v[8];
 #pragma unroll
-      for (int i = 0; i < 8; ++i) v[i] = q[min(z0 + i, nsplit - 1) * step + c];
+      for (int i = 0; i < 8; ++i) v[i] = q[min(z0 + i, n - 1) * step + c];
 #pragma unroll
-      for (int i = 0; i < 8; ++i) a = fmaf(__shfl(f_mine, min(z0 + i, 63)) * (z0 + i < nsplit ? 1.f : 0.f), v[i], a);
+      for (int i = 0; i < 8; ++i) a = fmaf(__shfl(f_mine, min(z0 + i, 63)) * (z0 + i < n ? 1.f : 0.f), v[i], a);
     }
     if (c0 + lane < Dv) st_f((T*)p.out + t * p.ldo + (long)h * Dv + c, a * inv);
   }

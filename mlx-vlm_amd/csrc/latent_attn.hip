@@ -9,7 +9,7 @@
 //
 //   vlm_latent_kv_write      d = W_dkv h rows -> c = d[:R] * rsqrt(mean(d[:R]^2) + eps) * w, kr = rope(d[R:], pos) into the
 //                            paged pool [page][64][R + Dr] (T-typed) of the token's sequence
-//   vlm_rope_pairs_rows      rotate the Dr-wide rotary part of every head's query into the fp32 query buffer behind the
+//   vlm_rope_pairs_rows      rotate the Dr-wide rotary part of every head's query into the (fp32 or T) query buffer behind the
 //                            absorbed part
 //                            (both: pairs (2 i, 2 i + 1), or with rot_half the pairs (i, i + Dr / 2))
 //   vlm_latent_attn          causal softmax attention of fp32 queries [T][H][R + Dr] over the pool, one workgroup per (token,
@@ -87,10 +87,10 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(const T* __restric
   }
 }
 
-template <typename T>
+template <typename T, typename TO>
 __global__ __launch_bounds__(256) void rope_pairs_rows_kernel(const T* __restrict__ q, long ldq, long head_stride, int H, int Dr,
                                                               const float* __restrict__ inv_freq, const int* __restrict__ tok_pos,
-                                                              float* __restrict__ out, long ldo, long out_head_stride, int rows,
+                                                              TO* __restrict__ out, long ldo, long out_head_stride, int rows,
                                                               int rot_half, float amp) {
   const long i = (long)blockIdx.x * 256 + threadIdx.x;
   const int hp = Dr / 2;
@@ -104,9 +104,9 @@ __global__ __launch_bounds__(256) void rope_pairs_rows_kernel(const T* __restric
   sincosf((float)tok_pos[t] * inv_freq[pi], &sn, &cs);
   sn *= amp;
   cs *= amp;
-  float* dst = out + t * ldo + (long)h * out_head_stride;
-  dst[i0] = u * cs - v * sn;
-  dst[i1] = v * cs + u * sn;
+  TO* dst = out + t * ldo + (long)h * out_head_stride;
+  st_f(dst + i0, u * cs - v * sn);
+  st_f(dst + i1, v * cs + u * sn);
 }
 
 // workgroup = (token, head): one key per lane and tile for the scores, one value dimension per lane for the weighted sum
@@ -473,18 +473,17 @@ extern "C" int vlm_latent_kv_write(const void* d, long ldd, const void* w, int R
 }
 
 extern "C" int vlm_rope_pairs_rows(const void* q, long ldq, long head_stride, int H, int Dr, const void* inv_freq, const void* tok_pos,
-                                   void* out, long ldo, long out_head_stride, int rot_half, float amp, int rows, int dtype,
+                                   void* out, long ldo, long out_head_stride, int rot_half, float amp, int out_f32, int rows, int dtype,
                                    void* stream) {
-  if (!q || !tok_pos || !out || H <= 0 || Dr < 0 || (Dr & 1) || (Dr && !inv_freq) || rows < 0) return VLM_ERR_ARG;
+  if (!q || !tok_pos || !out || H <= 0 || Dr < 0 || (Dr & 1) || (Dr && !inv_freq) || rows < 0 || (dtype && !out_f32)) return VLM_ERR_ARG;
   if (rows == 0 || Dr == 0) return VLM_OK;
   hipStream_t st = (hipStream_t)stream;
   const unsigned nb = (unsigned)(((long)rows * H * (Dr / 2) + 255) / 256);
-  if (dtype)
-    hipLaunchKernelGGL(rope_pairs_rows_kernel<float>, dim3(nb), dim3(256), 0, st, (const float*)q, ldq, head_stride, H, Dr,
-                       (const float*)inv_freq, (const int*)tok_pos, (float*)out, ldo, out_head_stride, rows, rot_half, amp);
-  else
-    hipLaunchKernelGGL(rope_pairs_rows_kernel<bf16_t>, dim3(nb), dim3(256), 0, st, (const bf16_t*)q, ldq, head_stride, H, Dr,
-                       (const float*)inv_freq, (const int*)tok_pos, (float*)out, ldo, out_head_stride, rows, rot_half, amp);
+#define GO(T, TO)                                                                                                                   \
+  hipLaunchKernelGGL((rope_pairs_rows_kernel<T, TO>), dim3(nb), dim3(256), 0, st, (const T*)q, ldq, head_stride, H, Dr, (const float*)inv_freq, \
+                     (const int*)tok_pos, (TO*)out, ldo, out_head_stride, rows, rot_half, amp)
+  if (dtype) GO(float, float); else if (out_f32) GO(bf16_t, float); else GO(bf16_t, bf16_t);
+#undef GO
   VLM_CHECK_LAUNCH();
   return VLM_OK;
 }

@@ -7,6 +7,8 @@
 // prompt was cut into steps.  With all three in fp32 this is the true 32-bit product of the float32 serving mode; with
 // fp32 C and `accumulate` it adds a projection straight onto an fp32 residual stream.
 //
+// bf16 A and W with aligned rows and more than 8 rows of A take the matrix cores instead (linear_any_mfma_kernel: fp32 sums in blocks of 32 k).
+//
 // 64 x 64 output tile per workgroup of 256 lanes (4 waves), 16-deep k slabs staged through LDS as fp32, 4 x 4 outputs
 // per lane.  Per-head projections of one tensor (latent attention's absorbed key / value maps) run as `batch` with
 // element strides between heads.
@@ -217,12 +219,97 @@ __global__ __launch_bounds__(256) void linear_rows_vec_kernel(const TA* __restri
   }
 }
 
+// bf16 operands of more than 8 rows whose rows come in whole 16-byte pieces, on v_mfma_f32_16x16x32_bf16 with fp32 sums: per-head maps as
+// batch and products with fp32 results (the GEMMs of gemm_bf16.hip write bf16).  A wave owns 32 rows of A x 64 rows of W, a workgroup
+// 64 x 128; operands come straight from global memory in the operand layout (the W rows of a tile are shared through the caches), a lane
+// ends with 4 neighbouring outputs of one row.
+template <typename TC>
+__global__ __launch_bounds__(256) void linear_any_mfma_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, TC* __restrict__ C, int M,
+                                                              int N, int K, long lda, long ldw, long ldc, long sA, long sW, long sC,
+                                                              int accumulate) {
+  typedef __attribute__((ext_vector_type(8))) __bf16 bf8;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, g = lane >> 4;
+  const int m0 = blockIdx.y * 64 + (wave & 1) * 32, n0 = blockIdx.x * 128 + (wave >> 1) * 64;
+  if (m0 >= M || n0 >= N) return;
+  A += (long)blockIdx.z * sA;
+  W += (long)blockIdx.z * sW;
+  C += (long)blockIdx.z * sC;
+  const bf16_t *ar[2], *wr[4];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) ar[i] = A + (long)min(m0 + 16 * i + r16, M - 1) * lda + 8 * g;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) wr[j] = W + (long)min(n0 + 16 * j + r16, N - 1) * ldw + 8 * g;
+  f32x4_t acc[2][4];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const int K32 = K & ~31;
+#pragma unroll 2
+  for (int k = 0; k < K32; k += 32) {
+    bf8 a[2], w[4];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) a[i] = *reinterpret_cast<const bf8*>(ar[i] + k);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) w[j] = *reinterpret_cast<const bf8*>(wr[j] + k);
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[j], a[i], acc[i][j], 0, 0, 0);
+  }
+  if (K32 < K) {
+    const u32x4_t none = {0u, 0u, 0u, 0u};
+    bf8 a[2], w[4];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) a[i] = __builtin_bit_cast(bf8, none);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) w[j] = __builtin_bit_cast(bf8, none);
+    if (K32 + 8 * g < K) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i) a[i] = *reinterpret_cast<const bf8*>(ar[i] + K32);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) w[j] = *reinterpret_cast<const bf8*>(wr[j] + K32);
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[j], a[i], acc[i][j], 0, 0, 0);
+  }
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int m = m0 + 16 * i + r16;
+    if (m >= M) continue;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int n = n0 + 16 * j + 4 * g;
+      TC* c = C + (long)m * ldc + n;
+      if (n + 4 <= N && !accumulate && (((uintptr_t)c) & (4 * sizeof(TC) - 1)) == 0) {
+        if constexpr (sizeof(TC) == 4) *reinterpret_cast<float4*>(c) = make_float4(acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]);
+        else *reinterpret_cast<uint2*>(c) = make_uint2(pack_bf2(acc[i][j][0], acc[i][j][1]), pack_bf2(acc[i][j][2], acc[i][j][3]));
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (n + r < N) st_f(c + r, accumulate ? ld_f(c + r) + acc[i][j][r] : acc[i][j][r]);
+      }
+    }
+  }
+}
+
 template <typename TA, typename TW, typename TC>
 int launch(const void* A, const void* W, void* C, int M, int N, int K, long lda, long ldw, long ldc, int batch, long sA, long sW,
            long sC, int accumulate, hipStream_t st) {
   // all-fp32 operands (the float32 serving mode) always take the tile kernel: one summation order for every row count, so a
   // token's result is the same bits in a prompt, in a portion and decoded alone
   constexpr bool all_f32 = sizeof(TA) == 4 && sizeof(TW) == 4 && sizeof(TC) == 4;
+  if constexpr (sizeof(TA) == 2 && sizeof(TW) == 2) {
+    if (M > 8 && K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && sA % 8 == 0 && sW % 8 == 0 && (((uintptr_t)A | (uintptr_t)W) & 15) == 0) {
+      dim3 grid((N + 127) / 128, (M + 63) / 64, batch);
+      hipLaunchKernelGGL((linear_any_mfma_kernel<TC>), grid, dim3(256), 0, st, (const bf16_t*)A, (const bf16_t*)W, (TC*)C, M, N, K, lda, ldw, ldc,
+                         sA, sW, sC, accumulate);
+      VLM_CHECK_LAUNCH();
+      return VLM_OK;
+    }
+  }
   if (M <= 8 && !all_f32) {
     dim3 grid((N + 3) / 4, 1, batch);
     hipLaunchKernelGGL((linear_rows_kernel<TA, TW, TC>), grid, dim3(256), 0, st, (const TA*)A, (const TW*)W, (TC*)C, M, N, K, lda,

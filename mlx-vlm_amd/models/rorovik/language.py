@@ -151,13 +151,17 @@ class LanguageModel(RaggedLanguageModel):
         cq = ops.latent_prep_rows(proj[:, ns.off["dkv"]:], ns.dkv_norm, R, Dr, ns.inv_freq, pl.tok_seq, pl.tok_pos, bt, cpool,
                                   self.config.norm_eps, amp=ns.amp, dq=proj[:, ns.off["dq"]:], wq=ns.dq_norm)
         q = self._linear(cq, ns.wuq)
-        qabs = torch.empty(Tn, H * (R + Dr), dtype=torch.float32, device=dev)
+        mfma = ops.latent_mfma_fits(cpool, R, Dr)
+        qabs = torch.empty(Tn, H * (R + Dr), dtype=torch.bfloat16 if mfma else torch.float32, device=dev)
         # absorbed keys: q'_h = U_k,h^T q_h for every head (batch = heads, strides inside the packed rows)
         ops.linear_any(q, ns.uk_t.view(H * R, D), out=qabs, M=Tn, N=R, K=D, batch=H, stride_a=D + Dr, stride_w=R * D, stride_c=R + Dr)
         if Dr:
             ops.rope_pairs_rows(q[:, D:], D + Dr, H, Dr, ns.inv_freq, pl.tok_pos, qabs[:, R:], R + Dr, amp=ns.amp)
         qv = qabs.view(Tn, H, R + Dr)
-        if (self.dtype == torch.float32 or Tn > self.ROWS_FORM) and R <= 512 and (32 * _al8(R + Dr) + 512) * 4 <= 150 * 1024:
+        if mfma:
+            ol = ops.latent_attn_mfma(qv, cpool, pl.tok_seq, pl.tok_pos, bt, H, R, Dr, ns.scale, sink=ns.sink,
+                                      blocks=None if Tn <= self.ROWS_FORM else (pl.qb_start, pl.qb_count))
+        elif (self.dtype == torch.float32 or Tn > self.ROWS_FORM) and R <= 512 and (32 * _al8(R + Dr) + 512) * 4 <= 150 * 1024:
             ol = ops.latent_attn_blocks(qv, cpool, pl.qb_start, pl.qb_count, pl.tok_seq, pl.tok_pos, bt, H, R, Dr, ns.scale, sink=ns.sink)
         else:
             ol = ops.latent_attn(qv, cpool, pl.tok_seq, pl.tok_pos, bt, H, R, Dr, ns.scale, sink=ns.sink)

@@ -677,7 +677,7 @@ def rope_pairs_rows(q, head_stride, H, Dr, inv_freq, tok_pos, out, out_head_stri
     are 2-D views at the part's first column"""
     _dev(q, inv_freq, tok_pos, out)
     check(_lib.lib().vlm_rope_pairs_rows(_p(q), q.stride(0), int(head_stride), int(H), int(Dr), _p(inv_freq), _p(tok_pos), _p(out),
-                                         out.stride(0), int(out_head_stride), int(bool(rot_half)), float(amp), q.shape[0], _f32(q), _stream()),
+                                         out.stride(0), int(out_head_stride), int(bool(rot_half)), float(amp), _f32(out), q.shape[0], _f32(q), _stream()),
           "rope_pairs_rows")
 
 
@@ -712,6 +712,39 @@ def latent_attn_blocks(q, pool, qb_start, qb_count, tok_seq, tok_pos, block_tabl
                                             _p(block_table), block_table.shape[1], int(H), int(R), int(Dr), float(scale), int(window),
                                             _p(sink), _p(gate), gate.stride(0) if gate is not None else 0, _p(out), _f32(pool), _stream()),
           "latent_attn_blocks")
+    return out
+
+
+def latent_mfma_fits(pool, R, Dr):
+    """whether the matrix-core forms of the latent attention take these rows"""
+    return pool.dtype == torch.bfloat16 and R % 8 == 0 and Dr % 8 == 0 and R <= 512 and R + Dr <= 576
+
+
+def latent_attn_mfma(q, pool, tok_seq, tok_pos, block_table, H, R, Dr, scale, blocks=None, gate=None, out=None, window=0, sink=None, nsplit=None):
+    """latent attention on the bf16 matrix cores (see latent_mfma_fits): q bf16 [T, H, R + Dr] over a bf16 pool -> bf16 [T, H, R].
+    blocks = (qb_start, qb_count): the prompt form over query blocks, else the decode form (nsplit workgroups share a token's keys)"""
+    qb, qc = blocks if blocks is not None else (None, None)
+    _dev(q, pool, tok_seq, tok_pos, block_table, gate, out, sink, qb, qc)
+    _sink_ok(sink, H)
+    T = q.shape[0]
+    if q.dtype != torch.bfloat16 or not q.is_contiguous() or q.numel() != T * H * (R + Dr) or tok_seq.numel() != T or pool.dtype != torch.bfloat16 \
+            or pool.shape[-1] != R + Dr or not pool.is_contiguous() or (gate is not None and gate.dtype != torch.bfloat16):
+        raise _lib.VlmHipError("latent_attn_mfma: bf16 queries [T, H, R + Dr], a bf16 pool of rows [R + Dr], bf16 gates expected")
+    if out is None:
+        out = torch.empty(T, H, R, dtype=torch.bfloat16, device=q.device)
+    a = _lib.LatentMfmaArgs()
+    a.q, a.pool, a.tok_seq, a.tok_pos, a.block_table, a.max_pages = _p(q), _p(pool), _p(tok_seq), _p(tok_pos), _p(block_table), block_table.shape[1]
+    a.H, a.R, a.Dr, a.scale, a.window, a.sink = int(H), int(R), int(Dr), float(scale), int(window), _p(sink)
+    a.gate, a.ldgate, a.out = _p(gate), gate.stride(0) if gate is not None else 0, _p(out)
+    if blocks is not None:
+        a.qb_start, a.qb_count = _p(qb), _p(qc)
+        check(_lib.lib().vlm_latent_attn_mfma_blocks(C.byref(a), qb.numel(), _stream()), "latent_attn_mfma_blocks")
+        return out
+    span = min(block_table.shape[1] * 64, window if window > 0 else 1 << 30)              # keys a query can see
+    nsplit = max(1, min(256 // max(T * -(-H // 16), 1), -(-span // 128), 32)) if nsplit is None else int(nsplit)
+    part = torch.empty(nsplit, H, T, R + 2, dtype=torch.float32, device=q.device) if nsplit > 1 else None
+    a.nsplit, a.part = nsplit, _p(part)
+    check(_lib.lib().vlm_latent_attn_mfma_rows(C.byref(a), T, _stream()), "latent_attn_mfma_rows")
     return out
 
 
