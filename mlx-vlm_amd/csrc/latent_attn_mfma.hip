@@ -45,8 +45,9 @@ template <int NKS> __device__ __forceinline__ void load_queries(const bf16_t* qr
 // copies of a page's rows into a tile by 256 threads: this thread's pieces are tid, tid + 256, ... (a page's rows are contiguous in memory);
 // rows past the last key repeat its last piece (they are masked)
 template <int NKS> struct Stager {
+  static constexpr int HALF = NKS / 2;                   // a page goes through the registers in two halves
   int loff[NKS], pieces, D8;
-  u32x4_t st[NKS];
+  u32x4_t st[HALF];
   __device__ __forceinline__ void init(bf16_t* tiles, int ntiles, int Dk, int tid) {
     D8 = Dk / 8;
     pieces = PAGE * D8;
@@ -61,15 +62,15 @@ template <int NKS> struct Stager {
       *reinterpret_cast<u32x4_t*>(tiles + (i / (pad * PAGE)) * Tile<NKS>::SIZE + row * Tile<NKS>::PITCH + (D8 + i % pad) * 8) = u32x4_t{0u, 0u, 0u, 0u};
     }
   }
-  __device__ __forceinline__ void load(const bf16_t* page, int keys, int tid) {
+  template <int H> __device__ __forceinline__ void load(const bf16_t* page, int keys, int tid) {
     const u32x4_t* src = reinterpret_cast<const u32x4_t*>(page);
     const int have = min(pieces, keys * D8) - 1;
 #pragma unroll
-    for (int i = 0; i < NKS; ++i) st[i] = src[min(tid + 256 * i, have)];
+    for (int i = 0; i < HALF; ++i) st[i] = src[min(tid + 256 * (H * HALF + i), have)];
   }
-  __device__ __forceinline__ void store(bf16_t* tile) {
+  template <int H> __device__ __forceinline__ void store(bf16_t* tile) {
 #pragma unroll
-    for (int i = 0; i < NKS; ++i) *reinterpret_cast<u32x4_t*>(tile + loff[i]) = st[i];
+    for (int i = 0; i < HALF; ++i) *reinterpret_cast<u32x4_t*>(tile + loff[H * HALF + i]) = st[i];
   }
 };
 
@@ -95,15 +96,29 @@ __device__ __forceinline__ float softmax_update(float* pr, float& mrun, float& l
 
 // O^T += V^T P^T for 32 keys and 128 value columns: rows of this lane's 8 keys, 8 columns each (16 bytes)
 __device__ __forceinline__ void accumulate128(const u32x4_t* v, bf8 ph, bf8 pl, f32x4_t* acc) {
+  bf8 vt[8];
 #pragma unroll
   for (int b = 0; b < 8; ++b) {
     u32x4_t t;
 #pragma unroll
     for (int i = 0; i < 4; ++i) t[i] = pair_cols(v[2 * i][b / 2], v[2 * i + 1][b / 2], b & 1);
-    const bf8 vt = __builtin_bit_cast(bf8, t);
-    acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pl, acc[b], 0, 0, 0);
-    acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, ph, acc[b], 0, 0, 0);
+    vt[b] = __builtin_bit_cast(bf8, t);
+    acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt[b], pl, acc[b], 0, 0, 0);
   }
+#pragma unroll
+  for (int b = 0; b < 8; ++b) acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt[b], ph, acc[b], 0, 0, 0);
+  // the interleaving of the next column runs beside a product
+#pragma unroll
+  for (int b = 0; b < 8; ++b) {
+    __builtin_amdgcn_sched_group_barrier(0x2, 4, 0);     // VALU
+    __builtin_amdgcn_sched_group_barrier(0x8, 1, 0);     // MFMA
+  }
+  __builtin_amdgcn_sched_group_barrier(0x8, 8, 0);
+}
+// this lane's pieces of 8 keys (the contraction order of 32 keys from row `key0` on) at the columns from `cols` on
+__device__ __forceinline__ void load_values(const bf16_t* tile, int pitch, int key0, int cols, int r16, int g, u32x4_t* v) {
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = *reinterpret_cast<const u32x4_t*>(tile + (key0 + 16 * (i / 4) + 4 * g + i % 4) * pitch + cols + r16 * 8);
 }
 
 __device__ __forceinline__ float head_gate(const vlm_latent_mfma_args& p, long tok, int h) {
@@ -127,7 +142,7 @@ __global__ __launch_bounds__(256, 1) void latent_block_mfma_kernel(vlm_latent_mf
   const int first = window > 0 ? max(0, pos0 - window + 1) / PAGE : 0, tiles = last / PAGE + 1;
   Stager<NKS> sg;
   sg.init(tile, 2, Dk, tid);
-  sg.load(pool + (long)bt[first] * PAGE * Dk, last - first * PAGE + 1, tid);
+  sg.template load<0>(pool + (long)bt[first] * PAGE * Dk, last - first * PAGE + 1, tid);
   bf8 q[NKS];
   load_queries<NKS>((const bf16_t*)p.q + ((long)(t0 + r16) * p.H + h) * Dk, live && r16 < nq, Dk, g, q);
   f32x4_t acc[NVC][8];
@@ -136,19 +151,38 @@ __global__ __launch_bounds__(256, 1) void latent_block_mfma_kernel(vlm_latent_mf
 #pragma unroll
     for (int b = 0; b < 8; ++b) acc[c][b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float mrun = -INFINITY, lrun = 0.f;
-  sg.store(tile);
+  sg.template store<0>(tile);
+  sg.template load<1>(pool + (long)bt[first] * PAGE * Dk, last - first * PAGE + 1, tid);
+  sg.template store<1>(tile);
   for (int j = first; j < tiles; ++j) {
     const bf16_t* cur = tile + ((j - first) & 1) * TS;
+    bf16_t* nxt = tile + ((j + 1 - first) & 1) * TS;
+    const bool more = j + 1 < tiles;
+    const bf16_t* npage = pool + (long)bt[more ? j + 1 : j] * PAGE * Dk;
+    const int nkeys = last - (j + 1) * PAGE + 1;
     __syncthreads();                                     // the tile is written, and everybody is through with the other buffer
-    if (j + 1 < tiles) sg.load(pool + (long)bt[j + 1] * PAGE * Dk, last - (j + 1) * PAGE + 1, tid);
+    if (more) sg.template load<0>(npage, nkeys, tid);
+    // scores: two k steps of the four 16-key groups per batch, the next batch's reads ahead of this one's products
     f32x4_t s[4];
 #pragma unroll
     for (int u = 0; u < 4; ++u) s[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    bf8 ka[2][8];
+    auto keys = [&](int b, bf8* k) {
 #pragma unroll
-    for (int k = 0; k < NKS; ++k)
+      for (int i = 0; i < 8; ++i) k[i] = *reinterpret_cast<const bf8*>(cur + (16 * (i & 3) + r16) * KP + 32 * (2 * b + i / 4) + 8 * g);
+    };
+    keys(0, ka[0]);
 #pragma unroll
-      for (int u = 0; u < 4; ++u)
-        s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf8*>(cur + (16 * u + r16) * KP + 32 * k + 8 * g), q[k], s[u], 0, 0, 0);
+    for (int b = 0; b < NKS / 2; ++b) {
+      if (b + 1 < NKS / 2) keys(b + 1, ka[(b + 1) & 1]);
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s[i & 3] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[b & 1][i], q[2 * b + i / 4], s[i & 3], 0, 0, 0);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    u32x4_t v[2][8];
+    load_values(cur, KP, 0, 0, r16, g, v[0]);            // (in flight during the softmax)
+    __builtin_amdgcn_sched_barrier(0);
     const int lo = j * PAGE;
     float pr[16];
 #pragma unroll
@@ -167,19 +201,21 @@ __global__ __launch_bounds__(256, 1) void latent_block_mfma_kernel(vlm_latent_mf
 #pragma unroll
         for (int b = 0; b < 8; ++b) acc[c][b] *= al;
     }
-#pragma unroll
-    for (int kk = 0; kk < 2; ++kk) {
-      bf8 ph, pl;
-      split8(pr + 8 * kk, ph, pl);
-#pragma unroll
-      for (int c = 0; c < NVC; ++c) {
-        u32x4_t v[8];
-#pragma unroll
-        for (int i = 0; i < 8; ++i) v[i] = *reinterpret_cast<const u32x4_t*>(cur + (32 * kk + 16 * (i / 4) + 4 * g + i % 4) * KP + 128 * c + r16 * 8);
-        accumulate128(v, ph, pl, acc[c]);
-      }
+    if (more) {
+      sg.template store<0>(nxt);
+      sg.template load<1>(npage, nkeys, tid);
     }
-    if (j + 1 < tiles) sg.store(tile + ((j + 1 - first) & 1) * TS);
+    bf8 ph[2], pl[2];
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) split8(pr + 8 * kk, ph[kk], pl[kk]);
+#pragma unroll
+    for (int i = 0; i < 2 * NVC; ++i) {                  // 32 keys x 128 columns at a time, the next piece's reads ahead
+      if (i + 1 < 2 * NVC) load_values(cur, KP, 32 * ((i + 1) / NVC), 128 * ((i + 1) % NVC), r16, g, v[(i + 1) & 1]);
+      __builtin_amdgcn_sched_barrier(0);
+      accumulate128(v[i & 1], ph[i / NVC], pl[i / NVC], acc[i % NVC]);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    if (more) sg.template store<1>(nxt);
   }
   float l = col4_sum(lrun);
   const float ms = mrun == -INFINITY ? 0.f : mrun;
@@ -220,9 +256,10 @@ __global__ __launch_bounds__(256) void latent_rows_mfma_kernel(vlm_latent_mfma_a
     return;
   }
   const bf16_t* pool = (const bf16_t*)p.pool;
-  Stager<NKS> sg;
+  Stager<NKS> sg, sg2;                                   // (both halves of a page in flight at once)
   sg.init(tile, 1, Dk, tid);
-  sg.load(pool + (long)bt[first + z] * PAGE * Dk, pos - (first + z) * PAGE + 1, tid);
+  sg2.pieces = sg.pieces;
+  sg2.D8 = sg.D8;
   bf8 q[NKS];
   load_queries<NKS>((const bf16_t*)p.q + ((long)t * p.H + h0 + r16) * Dk, r16 < ncol, Dk, g, q);
   f32x4_t acc[8];
@@ -230,11 +267,14 @@ __global__ __launch_bounds__(256) void latent_rows_mfma_kernel(vlm_latent_mfma_a
   for (int b = 0; b < 8; ++b) acc[b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float mrun = -INFINITY, lrun = 0.f;
   for (int j = first + z; j < tiles; j += gridDim.z) {
+    const bf16_t* page = pool + (long)bt[j] * PAGE * Dk;
+    sg.template load<0>(page, pos - j * PAGE + 1, tid);
+    sg2.template load<1>(page, pos - j * PAGE + 1, tid);
     __syncthreads();                                     // (everybody is through with the previous page and its scores)
-    sg.store(tile);
+    sg.template store<0>(tile);
+#pragma unroll
+    for (int i = 0; i < NKS / 2; ++i) *reinterpret_cast<u32x4_t*>(tile + sg.loff[NKS / 2 + i]) = sg2.st[i];
     __syncthreads();
-    const int nx = j + gridDim.z;
-    if (nx < tiles) sg.load(pool + (long)bt[nx] * PAGE * Dk, pos - nx * PAGE + 1, tid);
     f32x4_t s = {0.f, 0.f, 0.f, 0.f};                    // keys 16 wave + 4 g + r of the page
 #pragma unroll
     for (int k = 0; k < NKS; ++k)
@@ -332,7 +372,7 @@ bool shape_ok(const vlm_latent_mfma_args* a) {
 #define LATENT_SIZES(GO)                                                        \
   do {                                                                          \
     const int Dk = a->R + a->Dr;                                                \
-    if (a->R <= 128 && Dk <= 160) GO(5, 1);                                     \
+    if (a->R <= 128 && Dk <= 192) GO(6, 1);                                     \
     else if (a->R <= 256 && Dk <= 320) GO(10, 2);                               \
     else GO(18, 4);                                                             \
   } while (0)
