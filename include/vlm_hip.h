@@ -708,6 +708,25 @@ int vlm_glu_rows(const void* g, long ldg, const void* u, long ldu, const void* r
  * ident fp32 [T].  E <= 256. */
 int vlm_moe_router_softmax(const void* h, long ldh, const void* w, long ldw, int D, int T, int E, int top, int identity,
                            const void* correction, void* gate, void* ident, int dtype, void* stream);
+/* csrc/moe_grouped.hip (ABI v14): experts of a prompt evaluated for the chosen (token, expert) pairs only.  vlm_moe_plan sorts the pairs by
+ * expert into slots, each expert's padded to whole tiles of 128: tok [cap] (-1: padding), tile_expert [cap / 128], ntiles [1], slots [T][top] (a
+ * token's slots in expert order, -1: fewer); cap >= (T * top rounded up to 128) + 128 E.  E <= 256. */
+int vlm_moe_plan(const void* gate, int T, int E, int top, int cap, void* tok, void* tile_expert, void* ntiles, void* slots, void* stream);
+typedef struct vlm_moe_grouped_args {
+  const void* a;                        /* up: bf16 rows [K] per TOKEN at lda; down: bf16 rows [ff] per SLOT at lda */
+  long lda;
+  const void* w;                        /* up: bf16 [E][gate rows ff | up rows ff][K] at ldw; down: bf16 [N][E * ff] at ldw */
+  long ldw;
+  const float* gate;                    /* up: fp32 [T][E] */
+  const int *tok, *tile_expert, *ntiles;
+  int E, ff, K, N;                      /* down: K = ff, N result columns */
+  int act;                              /* up: 0 tanh-form gelu, 1 silu, 3 clamped gate (as in vlm_glu_rows) */
+  float limit;
+  void* out;                            /* bf16 rows per SLOT at ldo: up act(g) * u * gate [ff], down [N]; padding slots are not written */
+  long ldo;
+} vlm_moe_grouped_args;
+int vlm_moe_grouped_up(const vlm_moe_grouped_args* a, int row_tiles, void* stream);     /* row_tiles = cap / 128; K % 64 == 0, ff % 8 == 0 */
+int vlm_moe_grouped_down(const vlm_moe_grouped_args* a, int row_tiles, void* stream);   /* ff % 64 == 0, N % 8 == 0 */
 int vlm_moe_relu2_gate(const void* up, long ldu, const void* gate, int E, int ff, int shared, void* out, long ldo, int rows, int dtype,
                        void* stream);
 
@@ -727,7 +746,7 @@ int vlm_scaled_add_rms(void* x, const void* y, long ldy, float mult, const void*
                        void* h, long ldh, int h_f32, int rows, int D, float eps, int dtype, void* stream);
 
 /* ABI v14.  The residual step of a sublayer that is normed before and after, fused with the next reader's norm:
- *   r = y[t] (+ bias) (+ pass[t] * src[t])     x[t] <- (init ? 0 : x[t]) + mult * rms(r) * wy     h[t] = rms(x[t]) * w, or T(x[t]) without w */
+ *   r = y[t] (or the sum of y[slots[t][k]]) (+ bias) (+ pass[t] * src[t])     x[t] <- (init ? 0 : x[t]) + mult * rms(r) * wy     h[t] = rms(x[t]) * w, or T(x[t]) without w */
 typedef struct vlm_sandwich_args {
   float* x;                             /* fp32 [rows][D] */
   int init;                             /* 1: x is written, not read */
@@ -735,6 +754,8 @@ typedef struct vlm_sandwich_args {
   int vocab;
   const void* y;                        /* T rows [D] at ldy */
   long ldy;
+  const int* slots;                     /* [rows][nslots] or NULL: the sum of the rows slots[t][k] of y instead of row t (negative: none) */
+  int nslots;
   const void* bias;                     /* T [D] or NULL */
   const float* pass;                    /* [rows] or NULL */
   const void* src;                      /* T rows [D] at ldsrc */

@@ -175,9 +175,15 @@ class LatentMfmaArgs(C.Structure):
 
 class SandwichArgs(C.Structure):
     """vlm_sandwich_args (include/vlm_hip.h)"""
-    _fields_ = [("x", c_void_p), ("init", c_int), ("ids", c_void_p), ("vocab", c_int), ("y", c_void_p), ("ldy", C.c_long), ("bias", c_void_p),
-                ("pass_", c_void_p), ("src", c_void_p), ("ldsrc", C.c_long), ("wy", c_void_p), ("mult", c_float), ("w", c_void_p),
+    _fields_ = [("x", c_void_p), ("init", c_int), ("ids", c_void_p), ("vocab", c_int), ("y", c_void_p), ("ldy", C.c_long),
+                ("slots", c_void_p), ("nslots", c_int), ("bias", c_void_p), ("pass_", c_void_p), ("src", c_void_p), ("ldsrc", C.c_long), ("wy", c_void_p), ("mult", c_float), ("w", c_void_p),
                 ("h", c_void_p), ("ldh", C.c_long), ("D", c_int), ("eps", c_float)]
+
+
+class MoeGroupedArgs(C.Structure):
+    """vlm_moe_grouped_args (include/vlm_hip.h)"""
+    _fields_ = ([("a", c_void_p), ("lda", C.c_long), ("w", c_void_p), ("ldw", C.c_long)] + [(n, c_void_p) for n in ("gate", "tok", "tile_expert", "ntiles")]
+                + [(n, c_int) for n in ("E", "ff", "K", "N", "act")] + [("limit", c_float), ("out", c_void_p), ("ldo", C.c_long)])
 
 
 class QkvRownormArgs(C.Structure):
@@ -311,6 +317,9 @@ SIGNATURES = {
                                        c_void_p, c_int, c_void_p]),
     "vlm_latent_attn_mfma_blocks": (c_int, [P(LatentMfmaArgs), c_int, c_void_p]),
     "vlm_latent_attn_mfma_rows": (c_int, [P(LatentMfmaArgs), c_int, c_void_p]),
+    "vlm_moe_plan": (c_int, [c_void_p] + [c_int] * 4 + [c_void_p] * 5),
+    "vlm_moe_grouped_up": (c_int, [P(MoeGroupedArgs), c_int, c_void_p]),
+    "vlm_moe_grouped_down": (c_int, [P(MoeGroupedArgs), c_int, c_void_p]),
     "vlm_sandwich_step": (c_int, [P(SandwichArgs), c_int, c_int, c_void_p]),
     "vlm_qkv_rownorm_rows": (c_int, [P(QkvRownormArgs), c_int, c_int, c_void_p]),
     "vlm_grouped_attn_blocks": (c_int, [P(GroupedAttnArgs), c_int, c_int, c_void_p]),

@@ -23,6 +23,7 @@
 //                              r = y[t] (+ bias) (+ pass[t] * src[t])                 (pass: weight of what the sublayer hands on of its input)
 //                              x[t] <- (init ? 0 : x[t]) + mult * r * rsqrt(mean(r^2) + eps) * wy
 //                              h[t] = x[t] * rsqrt(mean(x[t]^2) + eps) * w, or T(x[t]) without w, or nothing without h
+//                            With slots the first term is the sum of the rows y[slots[t][k]] (negative: none): experts evaluated pair by pair.
 //                            With ids the row y[ids[t]] is read instead of y[t] (a normed embedding lookup with init = 1, mult = 1).
 //   vlm_logit_cap_rows       out[t][j] = cap * tanh(scale * x[t][j] / cap)    (cap = 0: scale * x alone); x and out each fp32 or bf16, may be
 //                                                                                      the same rows
@@ -233,6 +234,7 @@ __global__ __launch_bounds__(256) void sandwich_kernel(vlm_sandwich_args p) {
     yr = id < 0 ? 0 : (id >= p.vocab ? p.vocab - 1 : id);
   }
   const T* y = (const T*)p.y + yr * p.ldy;
+  const int* slots = p.slots ? p.slots + t * p.nslots : nullptr;
   const T* src = p.pass ? (const T*)p.src + t * p.ldsrc : nullptr;
   const float pw = p.pass ? p.pass[t] : 0.f;
   float* xr = p.x + t * D;
@@ -244,7 +246,18 @@ __global__ __launch_bounds__(256) void sandwich_kernel(vlm_sandwich_args p) {
 #pragma unroll
     for (int j = 0; j < V; ++j) v[i][j] = xv[i][j] = 0.f;
     if (d < D) {
-      ldv<V>(y + d, v[i]);
+      if (slots) {
+        for (int k = 0; k < p.nslots; ++k) {
+          const int s = slots[k];
+          if (s < 0) continue;
+          float b[V];
+          ldv<V>((const T*)p.y + (long)s * p.ldy + d, b);
+#pragma unroll
+          for (int j = 0; j < V; ++j) v[i][j] += b[j];
+        }
+      } else {
+        ldv<V>(y + d, v[i]);
+      }
       if (!p.init) ldv<V>(xr + d, xv[i]);
       if (p.bias) {
         float b[V];
@@ -454,7 +467,7 @@ extern "C" int vlm_scaled_add_rms(void* x, const void* y, long ldy, float mult, 
 
 extern "C" int vlm_sandwich_step(const vlm_sandwich_args* a, int rows, int dtype, void* stream) {
   if (!a || !a->x || !a->y || !a->wy || !STREAM_ARGS_OK(rows, a->D) || a->ldy < a->D || (a->ids && a->vocab <= 0) ||
-      (a->pass && (!a->src || a->ldsrc < a->D)) || (a->h && a->ldh < a->D) || (a->w && !a->h))
+      (a->slots && (a->nslots <= 0 || a->ids)) || (a->pass && (!a->src || a->ldsrc < a->D)) || (a->h && a->ldh < a->D) || (a->w && !a->h))
     return VLM_ERR_ARG;
   if (rows == 0) return VLM_OK;
   hipStream_t st = (hipStream_t)stream;

@@ -12,4 +12,4 @@ from .rorovik import Model
 __all__ = ["Model", "ModelConfig", "LayerConfig", "LanguageModel"]
 
 # the operator sources (csrc/<name>.hip) the model's step function needs: what a trace replay of a fresh checkout compiles
-HIP_SOURCES = ('gemm_bf16', 'gemm256_bf16', 'linear_any', 'stream_f32', 'moe', 'latent_attn', 'latent_attn_mfma', 'grouped_attn')
+HIP_SOURCES = ('gemm_bf16', 'gemm256_bf16', 'linear_any', 'stream_f32', 'moe', 'moe_grouped', 'latent_attn', 'latent_attn_mfma', 'grouped_attn')

@@ -11,9 +11,10 @@ the next reader's input, one kernel:
                        absorbed form q' = U_k^T q per head straight over the cached rows, sink softmax, U_v per head; W_o
     x += m * norm1b(.)          and norm2 (or the next reader), one kernel
     dense ff  : h2 @ [gate | up]^T, relu(gate + b) * (up + b), W_down (its bias enters in the residual step)
-    moe ff    : router logits, softmax scores and choice in one kernel; ONE GEMM over every expert's [gate | up] rows, clamped gate * weight (exact
-                zeros for the experts a token did not choose), ONE GEMM over the stacked W_down - the sum over experts is its k loop;
-                identity experts add weight * h2 in the residual step
+    moe ff    : router logits, softmax scores and choice in one kernel; bf16 prompts: the chosen pairs sorted by expert, gathered [gate | up] products
+                with the clamped gate * weight, W_down per pair, summed in the residual step; other steps: ONE GEMM over every expert's
+                [gate | up] rows, clamped gate * weight (exact zeros for the experts a token did not choose), ONE GEMM over the
+                stacked W_down - the sum over experts is its k loop; identity experts add weight * h2 in the residual step
     x += m * norm2b(.)          and x in the serving dtype, one kernel
     token input: gelu_tanh(x @ side.gate^T) * side.embed[token, layer slice], side.proj
     x += m * rms(.) * side.norm and the next layer's norm1, one kernel
@@ -36,6 +37,7 @@ class LanguageModel(RaggedLanguageModel):
     NAME = "Rorovik"
     STATEFUL = False       # row caches only: a step that ran is taken back by moving the cache offset
     ROWS_FORM = 8          # steps of up to this many tokens run the decode form of the attentions
+    GROUPED_ROWS = 64      # bf16 steps of at least this many tokens evaluate only the chosen (token, expert) pairs
 
     def __init__(self, config: ModelConfig, **kwargs):
         super().__init__(config, **kwargs)
@@ -172,23 +174,29 @@ class LanguageModel(RaggedLanguageModel):
 
     # ------------------------------------------------------------------ feed-forwards
     def _feed_forward(self, ns, h, keep):
-        """-> (rows before the bias of the down projection, weight of the input rows handed on or None)"""
+        """-> what the residual step adds up: the result rows, and of experts the weight of the input rows handed on and, where the chosen pairs
+        were evaluated one by one, each token's rows"""
         Tn, T, dev, ff = h.shape[0], self.dtype, self.device, ns.ff
         if ns.moe:
             few = Tn <= self.STREAM_ROWS and T != torch.float32       # decode rows over bf16 weights: weight-streaming projections
             route, ident = ops.moe_router_softmax(h, ns.router, ns.top, ns.identity, ns.corr)
+            step = dict(pass_=ident, src=h) if ident is not None else {}
+            if Tn >= self.GROUPED_ROWS and ops.moe_grouped_fits(h, ns.wff, ns.down, ff):
+                y, slots = ops.moe_grouped_rows(h, ns.wff, ns.down, route, ns.top, ops.GLU_CLAMPED, ns.limit)
+                keep += [route, y, step]
+                return y, dict(step, slots=slots)
             gu = self._linear(h, ns.wff, skip=dict(skip_gate=route, skip_col0=0, E=ns.E, ff=2 * ff) if few else None)
             act = torch.empty(Tn, _al8(ns.E * ff), dtype=T, device=dev)[:, : ns.E * ff]
             ops.glu_rows(gu, gu[:, ff:], ops.GLU_CLAMPED, out=act, route=route, E=ns.E, ff=ff, estride=2 * ff, limit=ns.limit)
             keep.append(route)
         else:
-            ident = None
+            step = dict(bias=ns.down_b)
             gu = self._linear(h, ns.wff)
             act = torch.empty(Tn, _al8(ff), dtype=T, device=dev)[:, :ff]
             ops.glu_rows(gu[:, ns.foff["gate"]: ns.foff["gate"] + ff], gu[:, ns.foff["up"]:], ops.GLU_RELU, out=act, gbias=ns.gate_b, ubias=ns.up_b)
         y = self._linear(act, ns.down)
-        keep += [gu, act, y, ident]
-        return y, ident
+        keep += [gu, act, y, step]
+        return y, step
 
     # ------------------------------------------------------------------ the device side of a step
     def _run(self, pl, logits_dtype=torch.float32):
@@ -210,8 +218,8 @@ class LanguageModel(RaggedLanguageModel):
             h = ops.sandwich_step(x, y, ns.norm1b, mult, eps=eps, **(dict(w=ns.norm2) if ns.ff else last))
             if ns.ff:
                 h2 = h
-                y, ident = self._feed_forward(ns, h2, keep)
-                h = ops.sandwich_step(x, y, ns.norm2b, mult, eps=eps, bias=ns.down_b, pass_=ident, src=h2 if ident is not None else None, **last)
+                y, step = self._feed_forward(ns, h2, keep)
+                h = ops.sandwich_step(x, y, ns.norm2b, mult, eps=eps, **step, **last)
                 keep.append(h2)
             if side:
                 gt = self._linear(h, ns.side_gate)

@@ -807,14 +807,64 @@ def moe_router_softmax(h, w, top, identity=0, correction=None):
     return gate, ident
 
 
-def sandwich_step(x, y, wy, mult=1.0, w=None, eps=1e-6, bias=None, pass_=None, src=None, ids=None, init=False, h=None, cast=False):
+MOE_TILE = 128
+
+
+def moe_plan(gate, top):
+    """gate table fp32 [T, E] (at most `top` entries per row are not zero) -> the chosen pairs sorted by expert into slots (tok, tile_expert,
+    ntiles, slots [T, top]): see vlm_moe_plan"""
+    _dev(gate)
+    T, E = gate.shape
+    if gate.dtype != torch.float32 or not gate.is_contiguous():
+        raise _lib.VlmHipError("moe_plan: contiguous fp32 gate table expected")
+    tiles = -(-T * top // MOE_TILE) + E
+    dev, i32 = gate.device, torch.int32
+    tok = torch.empty(tiles * MOE_TILE, dtype=i32, device=dev)
+    tile_expert, ntiles = torch.empty(tiles, dtype=i32, device=dev), torch.empty(1, dtype=i32, device=dev)
+    slots = torch.empty(T, top, dtype=i32, device=dev)
+    check(_lib.lib().vlm_moe_plan(_p(gate), T, E, int(top), tiles * MOE_TILE, _p(tok), _p(tile_expert), _p(ntiles), _p(slots), _stream()), "moe_plan")
+    return tok, tile_expert, ntiles, slots
+
+
+def moe_grouped_fits(h, wup, wdown, ff):
+    """whether the pair-by-pair form takes these rows and stacked expert weights"""
+    return (h.dtype == torch.bfloat16 and wup.dtype == torch.bfloat16 and h.shape[1] % 64 == 0 and ff % 64 == 0 and wdown.shape[0] % 8 == 0
+            and h.stride(0) % 8 == 0 and wup.stride(0) % 8 == 0 and wdown.stride(0) % 8 == 0)
+
+
+def moe_grouped_rows(h, wup, wdown, gate, top, act, limit=float("inf")):
+    """rows h [T, K], experts' rows wup [E * 2 ff, K] ([gate_e | up_e] per expert), wdown [N, E * ff] (the experts' columns side by side), gate
+    fp32 [T, E] -> (bf16 rows [slots, N]: gate[t, e] * expert_e(h[t]) of every chosen pair, slots int32 [T, top] of each token, -1: fewer)"""
+    T, E = gate.shape
+    N, ff = wdown.shape[0], wdown.shape[1] // E
+    _dev(h, wup, wdown, gate)
+    if h.shape[0] != T or wup.shape[0] < E * 2 * ff or wup.shape[1] != h.shape[1] or wdown.shape[1] < E * ff or not moe_grouped_fits(h, wup, wdown, ff):
+        raise _lib.VlmHipError("moe_grouped_rows: bf16 rows and stacked expert weights with K and ff multiples of 64 expected")
+    tok, tile_expert, ntiles, slots = moe_plan(gate, top)
+    tiles = tile_expert.numel()
+    mid = torch.empty(tiles * MOE_TILE, ff, dtype=torch.bfloat16, device=h.device)
+    out = torch.empty(tiles * MOE_TILE, N, dtype=torch.bfloat16, device=h.device)
+    a = _lib.MoeGroupedArgs()
+    a.a, a.lda, a.w, a.ldw, a.gate = _p(h), h.stride(0), _p(wup), wup.stride(0), _p(gate)
+    a.tok, a.tile_expert, a.ntiles = _p(tok), _p(tile_expert), _p(ntiles)
+    a.E, a.ff, a.K, a.N, a.act, a.limit, a.out, a.ldo = E, ff, h.shape[1], N, int(act), float(limit), _p(mid), ff
+    check(_lib.lib().vlm_moe_grouped_up(C.byref(a), tiles, _stream()), "moe_grouped_up")
+    a.a, a.lda, a.w, a.ldw, a.K, a.out, a.ldo = _p(mid), ff, _p(wdown), wdown.stride(0), ff, _p(out), N
+    check(_lib.lib().vlm_moe_grouped_down(C.byref(a), tiles, _stream()), "moe_grouped_down")
+    return out, slots
+
+
+def sandwich_step(x, y, wy, mult=1.0, w=None, eps=1e-6, bias=None, pass_=None, src=None, ids=None, init=False, h=None, cast=False, slots=None):
     """r = y (+ bias) (+ pass_[t] * src[t]);  x <- (0 if init else x) + mult * rms(r) * wy;  returns h = rms(x) * w (or, with cast, x itself
-    in wy's dtype; None with neither).  ids: row ids[t] of the table y instead of row t.  x: contiguous fp32 [T, D], in place."""
-    _dev(x, y, wy, w, bias, pass_, src, ids, h)
+    in wy's dtype; None with neither).  ids: row ids[t] of the table y instead of row t; slots int32 [T, n]: the sum of the rows
+    y[slots[t, k]] (negative: none).  x: contiguous fp32 [T, D], in place."""
+    _dev(x, y, wy, w, bias, pass_, src, ids, h, slots)
     T, D = x.shape
     if x.dtype != torch.float32 or not x.is_contiguous() or y.dtype != wy.dtype or y.shape[1] < D or wy.numel() != D:
         raise _lib.VlmHipError("sandwich_step: contiguous fp32 stream, rows of its width in wy's dtype expected")
-    if (ids is None and y.shape[0] != T) or (ids is not None and (ids.dtype != torch.int32 or ids.numel() != T)):
+    if slots is not None and (slots.dtype != torch.int32 or slots.shape[0] != T or not slots.is_contiguous() or ids is not None):
+        raise _lib.VlmHipError("sandwich_step: contiguous int32 slots per stream row expected")
+    if (ids is None and slots is None and y.shape[0] != T) or (ids is not None and (ids.dtype != torch.int32 or ids.numel() != T)):
         raise _lib.VlmHipError("sandwich_step: one row (or one int32 id) per stream row expected")
     if pass_ is not None and (pass_.dtype != torch.float32 or pass_.numel() != T or src is None or src.dtype != y.dtype or src.shape[0] != T):
         raise _lib.VlmHipError("sandwich_step: fp32 pass weight per row and source rows expected")
@@ -822,6 +872,8 @@ def sandwich_step(x, y, wy, mult=1.0, w=None, eps=1e-6, bias=None, pass_=None, s
         h = torch.empty(T, D, dtype=wy.dtype, device=x.device)
     a = _lib.SandwichArgs()
     a.x, a.init, a.ids, a.vocab, a.y, a.ldy, a.bias = _p(x), int(bool(init)), _p(ids), y.shape[0], _p(y), y.stride(0), _p(bias)
+    if slots is not None:
+        a.slots, a.nslots = _p(slots), slots.shape[1]
     if pass_ is not None:
         a.pass_, a.src, a.ldsrc = _p(pass_), _p(src), src.stride(0)
     a.wy, a.mult, a.w, a.h, a.ldh, a.D, a.eps = _p(wy), float(mult), _p(w), _p(h), h.stride(0) if h is not None else 0, D, float(eps)

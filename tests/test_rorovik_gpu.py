@@ -172,6 +172,55 @@ def test_gated_units_with_biases_and_with_a_route_table(T, ff, E):
         assert (out.cpu()[(route == 0).repeat_interleave(ff, 1)] == 0).all()
 
 
+@pytest.mark.parametrize("T,K,E,top,ff,N", [(300, 128, 5, 2, 64, 72), (70, 64, 3, 3, 128, 64), (64, 192, 40, 4, 64, 320), (513, 64, 1, 1, 64, 8), (257, 64, 6, 2, 192, 128)])
+@pytest.mark.parametrize("act", [0, 1, 3])
+def test_experts_evaluated_pair_by_pair(T, K, E, top, ff, N, act):
+    """the chosen pairs sorted by expert (unequal counts, an expert without tokens, tokens with fewer pairs than `top` and with none), gathered
+    products, and their sum in the residual step"""
+    from mlx_vlm_amd import ops
+
+    g = torch.Generator().manual_seed(T + E)
+    bf = torch.bfloat16
+    h, wup, wdown = torch.randn(T, K + 8, generator=g).to(bf), (torch.randn(E * 2 * ff, K, generator=g) / K ** 0.5).to(bf), (torch.randn(N, E * ff, generator=g) / ff ** 0.5).to(bf)
+    gate = torch.zeros(T, E)
+    for t in range(T):
+        n = int(torch.randint(0, top + 1, (1,), generator=g)) if t % 3 == 0 else top
+        pick = torch.randperm(E, generator=g)[:n]
+        if E > 2:
+            pick = pick[pick != 1]                                                  # expert 1 stays without tokens
+        gate[t, pick] = torch.rand(len(pick), generator=g) + 0.1
+    tok, tile_expert, ntiles, slots = (x.cpu() for x in ops.moe_plan(gate.cuda(), top))
+    n = int(ntiles)
+    assert n == sum(-(-int((gate[:, e] != 0).sum()) // 128) for e in range(E))
+    at = 0
+    for e in range(E):
+        mine = torch.nonzero(gate[:, e]).view(-1)
+        tiles = -(-len(mine) // 128)
+        assert (tile_expert[at: at + tiles] == e).all()
+        seg = tok[at * 128: (at + tiles) * 128]
+        assert torch.equal(seg[: len(mine)].long(), mine) and (seg[len(mine):] == -1).all()
+        at += tiles
+    for t in range(T):
+        s = [int(i) for i in slots[t] if i >= 0]
+        assert [int(tile_expert[i // 128]) for i in s] == torch.nonzero(gate[t]).view(-1).tolist() and all(int(tok[i]) == t for i in s)
+    limit = 0.9
+    out, slots = ops.moe_grouped_rows(h.cuda()[:, :K], wup.cuda(), wdown.cuda(), gate.cuda(), top, act, limit)
+    hd, want = h.double()[:, :K], torch.zeros(T, N, dtype=F64)
+    for e in range(E):
+        a, u = hd @ wup.double()[e * 2 * ff: e * 2 * ff + ff].T, hd @ wup.double()[e * 2 * ff + ff: (e + 1) * 2 * ff].T
+        m = O.clamped_glu(a, u, limit) if act == 3 else (O.gelu_tanh(a) if act == 0 else a * torch.sigmoid(a)) * u
+        want += gate[:, e:e + 1].double() * (m @ wdown.double()[:, e * ff: (e + 1) * ff].T)
+    x = torch.zeros(T, N).cuda()
+    got = torch.zeros(T, N, dtype=F64)
+    o, sl = out.cpu().double(), slots.cpu()
+    for k in range(top):
+        ok = sl[:, k] >= 0
+        got[ok] += o[sl[ok, k].long()]
+    assert (got - want).abs().max() < 2e-2 * want.abs().max()
+    ops.sandwich_step(x, out, torch.ones(N, dtype=bf).cuda(), eps=1e-3, slots=slots, init=True)
+    assert (x.cpu().double() - O.rms(got, 1e-3)).abs().max() < 1e-4
+
+
 @pytest.mark.parametrize("HQ,HK,D,Dv", [(4, 2, 12, 20), (3, 3, 7, 5), (12, 2, 128, 128), (1, 1, 1, 1)])
 @pytest.mark.parametrize("T", [torch.float32, torch.bfloat16])
 def test_projection_rows_norm_over_all_heads_multiplier_and_mixed_values(T, HQ, HK, D, Dv):
@@ -371,6 +420,7 @@ ONE = {"attention": [H.attention()], "attention_equal_heads": [H.attention(heads
        "latent_wide": [H.latent(heads=4, dim=64, rot_dim=32, vdim=48, kv_rank=264, q_rank=100, base=10000.0)],
        "latent_rank_520": [H.latent(heads=2, dim=16, rot_dim=8, vdim=16, kv_rank=520, q_rank=16, mlp=None)],
        "latent_odd_sizes": [H.latent(heads=3, dim=7, rot_dim=2, vdim=9, kv_rank=21, q_rank=11, mlp=H.dense(19))],
+       "moe_pair_by_pair": [H.attention(mlp=H.moe(experts=6, identity=2, top=3, ff=64)), H.latent(mlp=H.moe(experts=4, identity=0, top=2, ff=128, limit=None))],
        "moe_all_chosen": [H.latent(mlp=H.moe(experts=3, identity=2, top=5))], "moe_top_1": [H.latent(mlp=H.moe(experts=7, identity=3, top=1, ff=9, limit=0.4))],
        "moe_mostly_identity": [H.attention(mlp=H.moe(experts=1, identity=6, top=3))]}
 
@@ -378,13 +428,15 @@ ONE = {"attention": [H.attention()], "attention_equal_heads": [H.attention(heads
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("kind", sorted(ONE))
 def test_each_mixer_and_feed_forward_alone(tmp_path, kind, dtype):
-    cfg = H.config(ONE[kind], side=0 if "equal" in kind else 12, mult=1.0 if "wide" in kind else 0.6)
+    cfg = H.config(ONE[kind], width=128 if "pair" in kind else 56, side=0 if "equal" in kind else 12, mult=1.0 if "wide" in kind else 0.6)
     W = H.weights(cfg, seed=3)
     ids = _ids(150, cfg["vocab"], 5)
     lm = _load(tmp_path, cfg, W, dtype, tokens=512).language_model
     want = _oracle(cfg, W, ids)
     assert _close(_whole(lm, ids), want, dtype)
     assert _close(_portions(lm, ids, [70, 1, 2, 30]), want, dtype)
+    if "pair" in kind and dtype == "bfloat16":
+        assert lm.GROUPED_ROWS <= 70
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
