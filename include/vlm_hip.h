@@ -709,9 +709,10 @@ int vlm_glu_rows(const void* g, long ldg, const void* u, long ldu, const void* r
 int vlm_moe_router_softmax(const void* h, long ldh, const void* w, long ldw, int D, int T, int E, int top, int identity,
                            const void* correction, void* gate, void* ident, int dtype, void* stream);
 /* csrc/moe_grouped.hip (ABI v14): experts of a prompt evaluated for the chosen (token, expert) pairs only.  vlm_moe_plan sorts the pairs by
- * expert into slots, each expert's padded to whole tiles of 128: tok [cap] (-1: padding), tile_expert [cap / 128], ntiles [1], slots [T][top] (a
+ * expert into slots, each expert's padded to whole tiles of 128: count [E] (tokens per expert), tok [cap] (-1: padding), tile_expert [cap / 128], ntiles [1], slots [T][top] (a
  * token's slots in expert order, -1: fewer); cap >= (T * top rounded up to 128) + 128 E.  E <= 256. */
-int vlm_moe_plan(const void* gate, int T, int E, int top, int cap, void* tok, void* tile_expert, void* ntiles, void* slots, void* stream);
+int vlm_moe_plan(const void* gate, int T, int E, int top, int cap, void* count, void* tok, void* tile_expert, void* ntiles, void* slots,
+                 void* stream);
 typedef struct vlm_moe_grouped_args {
   const void* a;                        /* up: bf16 rows [K] per TOKEN at lda; down: bf16 rows [ff] per SLOT at lda */
   long lda;

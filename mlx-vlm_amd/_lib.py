@@ -317,7 +317,7 @@ SIGNATURES = {
                                        c_void_p, c_int, c_void_p]),
     "vlm_latent_attn_mfma_blocks": (c_int, [P(LatentMfmaArgs), c_int, c_void_p]),
     "vlm_latent_attn_mfma_rows": (c_int, [P(LatentMfmaArgs), c_int, c_void_p]),
-    "vlm_moe_plan": (c_int, [c_void_p] + [c_int] * 4 + [c_void_p] * 5),
+    "vlm_moe_plan": (c_int, [c_void_p] + [c_int] * 4 + [c_void_p] * 6),
     "vlm_moe_grouped_up": (c_int, [P(MoeGroupedArgs), c_int, c_void_p]),
     "vlm_moe_grouped_down": (c_int, [P(MoeGroupedArgs), c_int, c_void_p]),
     "vlm_sandwich_step": (c_int, [P(SandwichArgs), c_int, c_int, c_void_p]),

@@ -219,6 +219,119 @@ __global__ __launch_bounds__(256) void linear_rows_vec_kernel(const TA* __restri
   }
 }
 
+// The same for bf16 activations: the rows are staged in LDS once per workgroup, so that whether a lane's activations are zero is known without
+// a trip to memory and a wave has the loads of NB pieces of R weight rows in flight at once; products on v_dot2_f32_bf16.
+template <typename TC, int MB, int R, int NB>
+__global__ __launch_bounds__(256) void linear_rows_stream_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, TC* __restrict__ C, int M,
+                                                                 int N, int K, long lda, long ldw, long ldc, int accumulate,
+                                                                 const float* __restrict__ skip_gate, int skip_col0, int E, int ff) {
+  extern __shared__ __align__(16) unsigned as[];         // [MB][K / 2] (rows past M: not read)
+  typedef __bf16 bf2 __attribute__((ext_vector_type(2)));
+  const int tid = threadIdx.x, lane = tid & 63, K2 = K / 2;
+  const int n0 = (blockIdx.x * 4 + (tid >> 6)) * R;
+  bool dead[R];                                          // (wave-uniform)
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int n = n0 + r;
+    dead[r] = n >= N;
+    if (skip_gate && n >= skip_col0 && n < skip_col0 + E * ff) {
+      const int e = (n - skip_col0) / ff;
+      bool any = false;
+      for (int m = 0; m < M; ++m) any |= skip_gate[(long)m * E + e] != 0.f;
+      dead[r] |= !any;
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < MB; ++m)
+    if (m < M)
+      for (int i = tid; i < K / 8; i += 256)
+        reinterpret_cast<uint4*>(as + m * K2)[i] = *reinterpret_cast<const uint4*>(A + (long)m * lda + 8 * i);
+  __syncthreads();
+  const bf16_t* w[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) w[r] = W + (long)min(n0 + r, N - 1) * ldw;
+  bool all = true;
+#pragma unroll
+  for (int r = 0; r < R; ++r) all &= dead[r];
+  float acc[R][MB] = {};
+  if (!all) {
+    for (int k0 = lane * 8; k0 < K; k0 += 512 * NB) {
+      u32x4_t wv[NB][R];
+#pragma unroll
+      for (int b = 0; b < NB; ++b) {
+        const int k = k0 + 512 * b;
+        unsigned nz = 0u;
+        if (k < K) {
+#pragma unroll
+          for (int m = 0; m < MB; ++m)
+            if (m < M) {
+              const uint4 a = *reinterpret_cast<const uint4*>(as + m * K2 + k / 2);
+              nz |= (a.x | a.y | a.z | a.w) & 0x7fff7fffu;
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+          wv[b][r] = u32x4_t{0u, 0u, 0u, 0u};
+          if (nz && !dead[r]) wv[b][r] = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(w[r] + k));
+        }
+      }
+#pragma unroll
+      for (int b = 0; b < NB; ++b) {
+        const int k = min(k0 + 512 * b, K - 8);
+#pragma unroll
+        for (int m = 0; m < MB; ++m)
+          if (m < M) {
+            const u32x4_t a = *reinterpret_cast<const u32x4_t*>(as + m * K2 + k / 2);
+#pragma unroll
+            for (int r = 0; r < R; ++r)
+#pragma unroll
+              for (int i = 0; i < 4; ++i) {
+                const unsigned x = a[i], y = wv[b][r][i];          // (scalars first: a bit cast of a vector element reads element 0)
+                acc[r][m] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf2, x), __builtin_bit_cast(bf2, y), acc[r][m], false);
+              }
+          }
+      }
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    if (n0 + r >= N) break;
+#pragma unroll
+    for (int m = 0; m < MB; ++m) {
+      if (m >= M) break;
+      const float v = wave_sum(acc[r][m]);
+      if (lane == 0) {
+        TC* c = C + (long)m * ldc + n0 + r;
+        st_f(c, accumulate ? ld_f(c) + v : v);
+      }
+    }
+  }
+}
+
+template <typename TC>
+int launch_stream(const void* A, const void* W, void* C, int M, int N, int K, long lda, long ldw, long ldc, int accumulate, const void* skip_gate,
+                  int skip_col0, int E, int ff, hipStream_t st) {
+  const int MB = M <= 1 ? 1 : M <= 2 ? 2 : M <= 4 ? 4 : 8;
+  const size_t lds = (size_t)MB * K * sizeof(bf16_t);
+  const int R = N <= 4096 ? 1 : 2;
+  const dim3 grid((N + 4 * R - 1) / (4 * R));
+#define GO(MBV, RV, NBV)                                                                                                            \
+  do {                                                                                                                              \
+    if (lds > 48 * 1024) {                                                                                                          \
+      hipError_t e = hipFuncSetAttribute((const void*)linear_rows_stream_kernel<TC, MBV, RV, NBV>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
+      if (e != hipSuccess) return VLM_ERR_HIP + (int)e;                                                                             \
+    }                                                                                                                               \
+    hipLaunchKernelGGL((linear_rows_stream_kernel<TC, MBV, RV, NBV>), grid, dim3(256), lds, st, (const bf16_t*)A, (const bf16_t*)W, (TC*)C, M, N, K, \
+                       lda, ldw, ldc, accumulate, (const float*)skip_gate, skip_col0, E, ff);                                       \
+  } while (0)
+#define GO2(MBV, NBV) do { if (R == 1) GO(MBV, 1, NBV); else GO(MBV, 2, NBV); } while (0)
+  if (MB == 1) GO2(1, 4); else if (MB == 2) GO2(2, 4); else if (MB == 4) GO2(4, 4); else GO2(8, 4);
+#undef GO2
+#undef GO
+  VLM_CHECK_LAUNCH();
+  return VLM_OK;
+}
+
 // bf16 operands of more than 8 rows whose rows come in whole 16-byte pieces, on v_mfma_f32_16x16x32_bf16 with fp32 sums: per-head maps as
 // batch and products with fp32 results (the GEMMs of gemm_bf16.hip write bf16).  A wave owns 32 rows of A x 64 rows of W, a workgroup
 // 64 x 128; operands come straight from global memory in the operand layout (the W rows of a tile are shared through the caches), a lane
@@ -338,6 +451,10 @@ extern "C" int vlm_linear_rows_bf16w(const void* A, const void* W, void* C, int 
   if (skip_gate && (E <= 0 || ff <= 0 || skip_col0 < 0 || skip_col0 + (long)E * ff > N)) return VLM_ERR_ARG;
   if (K % 8 || ldw % 8 || ((uintptr_t)W & 15)) return VLM_ERR_SHAPE;
   hipStream_t st = (hipStream_t)stream;
+  const int MB = M <= 1 ? 1 : M <= 2 ? 2 : M <= 4 ? 4 : 8;
+  if (!a_f32 && lda % 8 == 0 && ((uintptr_t)A & 15) == 0 && (size_t)MB * K * sizeof(bf16_t) <= 80 * 1024)
+    return c_f32 ? launch_stream<float>(A, W, C, M, N, K, lda, ldw, ldc, accumulate, skip_gate, skip_col0, E, ff, st)
+                 : launch_stream<bf16_t>(A, W, C, M, N, K, lda, ldw, ldc, accumulate, skip_gate, skip_col0, E, ff, st);
   dim3 grid((N + 3) / 4);
 #define GO(TA, TC)                                                                                                              \
   hipLaunchKernelGGL((linear_rows_vec_kernel<TA, TC>), grid, dim3(256), 0, st, (const TA*)A, (const bf16_t*)W, (TC*)C, M, N, K, lda, \

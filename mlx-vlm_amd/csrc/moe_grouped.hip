@@ -3,7 +3,7 @@
 // expert:
 //
 //   vlm_moe_plan          gate table fp32 [T][E] (0: not chosen) -> slot tables: tok [cap] (the slot's token, -1: padding), tile_expert [cap / 128],
-//                         ntiles, and per token its slots in expert order (slots [T][top], -1: fewer).  One workgroup.
+//                         ntiles, and per token its slots in expert order (slots [T][top], -1: fewer); count [E]: scratch
 //   vlm_moe_grouped_up    act[slot] = act(W_gate,e h[tok]) * (W_up,e h[tok]) * gate[tok][e]: gathered rows, both products and the activation in one
 //                         kernel.  W: expert e's rows [gate_e | up_e], 2 ff rows side by side
 //   vlm_moe_grouped_down  y[slot] = W_down,e act[slot]; W: the experts' columns side by side ([N][E ff])
@@ -22,53 +22,63 @@ constexpr int BM = 128, BN = 128, BK = 64, ROWB = BK * 2, STAGE = (BM + BN) * RO
 
 __device__ __forceinline__ int lds_off(int row, int slot) { return row * ROWB + ((slot ^ ((row >> 1) & 7)) << 4); }
 
-// one workgroup of 16 waves; wave w owns the experts w, w + 16, ...
-__global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict__ gate, int T, int E, int top, int cap, int* __restrict__ tok,
-                                                        int* __restrict__ tile_expert, int* __restrict__ ntiles, int* __restrict__ slots) {
-  __shared__ int cnt[256], base[257];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-  for (int e = wave; e < E; e += 16) {
-    int n = 0;
-#pragma unroll 4
-    for (int t0 = 0; t0 < T; t0 += 64) {
-      const int t = t0 + lane;
-      n += __popcll(__ballot(t < T && gate[(long)min(t, T - 1) * E + e] != 0.f));
-    }
-    if (lane == 0) cnt[e] = n;
-  }
+// grid (E): tokens of every expert; token slots marked empty
+__global__ __launch_bounds__(1024) void moe_count_kernel(const float* __restrict__ gate, int T, int E, int top, int* __restrict__ count,
+                                                         int* __restrict__ slots) {
+  __shared__ int part[16];
+  const int tid = threadIdx.x, e = blockIdx.x;
+  int n = 0;
+  for (int t = tid; t < T; t += 1024) n += gate[(long)t * E + e] != 0.f;
+  for (int i = e * 1024 + tid; i < T * top; i += E * 1024) slots[i] = -1;
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) n += __shfl_xor(n, o);
+  if ((tid & 63) == 0) part[tid >> 6] = n;
   __syncthreads();
   if (tid == 0) {
-    int b = 0;
-    for (int e = 0; e < E; ++e) {
-      base[e] = b;
-      b += (cnt[e] + BM - 1) / BM * BM;
-    }
-    base[E] = b;
-    *ntiles = b / BM;
+    int s = 0;
+    for (int w = 0; w < 16; ++w) s += part[w];
+    count[e] = s;
   }
+}
+
+// grid (E): the expert's first slot from the counts of those before it, then its tokens in order, 1024 at a time
+__global__ __launch_bounds__(1024) void moe_place_kernel(const float* __restrict__ gate, int T, int E, int top, const int* __restrict__ count,
+                                                         int* __restrict__ tok, int* __restrict__ tile_expert, int* __restrict__ ntiles,
+                                                         int* __restrict__ slots) {
+  __shared__ int part[16], before[16];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, e = blockIdx.x;
+  int b = 0;
+  for (int f = tid; f < e; f += 1024) b += (count[f] + BM - 1) / BM * BM;
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) b += __shfl_xor(b, o);
+  if (lane == 0) before[wave] = b;
   __syncthreads();
-  for (int i = tid; i < T * top; i += 1024) slots[i] = -1;
-  __threadfence_block();
-  __syncthreads();
-  for (int e = wave; e < E; e += 16) {
-    int at = base[e];
-    const int end = base[e + 1];
-    for (int i = at / BM + lane; i < end / BM; i += 64) tile_expert[i] = e;
-    for (int i = at + cnt[e] + lane; i < end; i += 64) tok[i] = -1;
-#pragma unroll 4
-    for (int t0 = 0; t0 < T; t0 += 64) {
-      const int t = t0 + lane;
-      const bool mine = t < T && gate[(long)min(t, T - 1) * E + e] != 0.f;
-      const unsigned long long m = __ballot(mine);
-      if (mine) {
-        const int slot = at + __popcll(m & ((1ull << lane) - 1ull));
-        int k = 0;                                       // how many experts before this one the token chose
-        for (int f = 0; f < e; ++f) k += gate[(long)t * E + f] != 0.f;
-        tok[slot] = t;
-        if (k < top) slots[(long)t * top + k] = slot;
-      }
-      at += __popcll(m);
+  int at = 0;
+  for (int w = 0; w < 16; ++w) at += before[w];
+  const int n = count[e], end = at + (n + BM - 1) / BM * BM;
+  if (e == E - 1 && tid == 0) *ntiles = end / BM;
+  for (int i = at / BM + tid; i < end / BM; i += 1024) tile_expert[i] = e;
+  for (int i = at + n + tid; i < end; i += 1024) tok[i] = -1;
+  for (int t0 = 0; t0 < T; t0 += 1024) {
+    const int t = t0 + tid;
+    const bool mine = t < T && gate[(long)min(t, T - 1) * E + e] != 0.f;
+    const unsigned long long m = __ballot(mine);
+    if (lane == 0) part[wave] = __popcll(m);
+    __syncthreads();
+    int ahead = 0, total = 0;
+    for (int w = 0; w < 16; ++w) {
+      if (w < wave) ahead += part[w];
+      total += part[w];
     }
+    if (mine) {
+      const int slot = at + ahead + __popcll(m & ((1ull << lane) - 1ull));
+      int k = 0;                                         // how many experts before this one the token chose
+      for (int f = 0; f < e; ++f) k += gate[(long)t * E + f] != 0.f;
+      tok[slot] = t;
+      if (k < top) slots[(long)t * top + k] = slot;
+    }
+    at += total;
+    __syncthreads();
   }
 }
 
@@ -203,11 +213,16 @@ template <bool UP> int grouped(const vlm_moe_grouped_args* a, int row_tiles, voi
 
 }  // namespace
 
-extern "C" int vlm_moe_plan(const void* gate, int T, int E, int top, int cap, void* tok, void* tile_expert, void* ntiles, void* slots, void* stream) {
-  if (!gate || !tok || !tile_expert || !ntiles || !slots || T <= 0 || E <= 0 || top <= 0 || (long)cap < ((long)T * top + BM - 1) / BM * BM + (long)E * BM)
+extern "C" int vlm_moe_plan(const void* gate, int T, int E, int top, int cap, void* count, void* tok, void* tile_expert, void* ntiles, void* slots,
+                            void* stream) {
+  if (!gate || !count || !tok || !tile_expert || !ntiles || !slots || T <= 0 || E <= 0 || top <= 0 ||
+      (long)cap < ((long)T * top + BM - 1) / BM * BM + (long)E * BM)
     return VLM_ERR_ARG;
-  if (E > 256) return VLM_ERR_SHAPE;
-  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), 0, (hipStream_t)stream, (const float*)gate, T, E, top, cap, (int*)tok, (int*)tile_expert,
+  if (E > 256 || (long)T * top > 0x3fffffff) return VLM_ERR_SHAPE;
+  hipStream_t st = (hipStream_t)stream;
+  hipLaunchKernelGGL(moe_count_kernel, dim3(E), dim3(1024), 0, st, (const float*)gate, T, E, top, (int*)count, (int*)slots);
+  VLM_CHECK_LAUNCH();
+  hipLaunchKernelGGL(moe_place_kernel, dim3(E), dim3(1024), 0, st, (const float*)gate, T, E, top, (const int*)count, (int*)tok, (int*)tile_expert,
                      (int*)ntiles, (int*)slots);
   VLM_CHECK_LAUNCH();
   return VLM_OK;

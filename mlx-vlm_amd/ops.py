@@ -821,8 +821,8 @@ def moe_plan(gate, top):
     dev, i32 = gate.device, torch.int32
     tok = torch.empty(tiles * MOE_TILE, dtype=i32, device=dev)
     tile_expert, ntiles = torch.empty(tiles, dtype=i32, device=dev), torch.empty(1, dtype=i32, device=dev)
-    slots = torch.empty(T, top, dtype=i32, device=dev)
-    check(_lib.lib().vlm_moe_plan(_p(gate), T, E, int(top), tiles * MOE_TILE, _p(tok), _p(tile_expert), _p(ntiles), _p(slots), _stream()), "moe_plan")
+    slots, count = torch.empty(T, top, dtype=i32, device=dev), torch.empty(E, dtype=i32, device=dev)
+    check(_lib.lib().vlm_moe_plan(_p(gate), T, E, int(top), tiles * MOE_TILE, _p(count), _p(tok), _p(tile_expert), _p(ntiles), _p(slots), _stream()), "moe_plan")
     return tok, tile_expert, ntiles, slots
 
 
