@@ -132,8 +132,8 @@ __global__ __launch_bounds__(256, 1) void latent_block_mfma_kernel(vlm_latent_mf
   extern __shared__ __align__(16) bf16_t tile[];         // [2][TS]
   const int R = p.R, Dk = p.R + p.Dr;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r16 = lane & 15, g = lane >> 4;
-  const int blk = gridDim.x - 1 - blockIdx.x;            // (the blocks of a prompt's end have the most keys: they start first)
-  const int t0 = p.qb_start[blk], nq = p.qb_count[blk], h = blockIdx.y * 4 + wave;
+  const int blk = gridDim.y - 1 - blockIdx.y;            // (the blocks of a prompt's end have the most keys: they start first)
+  const int t0 = p.qb_start[blk], nq = p.qb_count[blk], h = blockIdx.x * 4 + wave;
   const bool live = h < p.H;                             // (a wave without a head still helps with the loads)
   const int* bt = p.block_table + (long)p.tok_seq[t0] * p.max_pages;
   const int pos0 = p.tok_pos[t0], last = pos0 + nq - 1, mypos = r16 < nq ? pos0 + r16 : -1, window = p.window;
@@ -388,7 +388,8 @@ extern "C" int vlm_latent_attn_mfma_blocks(const vlm_latent_mfma_args* a, int nb
   if (bad(a) || !a->qb_start || !a->qb_count || nblocks < 0) return VLM_ERR_ARG;
   if (!shape_ok(a)) return VLM_ERR_SHAPE;
   if (nblocks == 0) return VLM_OK;
-  const dim3 grid(nblocks, (a->H + 3) / 4);
+  if (nblocks > 65535) return VLM_ERR_SHAPE;
+  const dim3 grid((a->H + 3) / 4, nblocks);
 #define GO(NKS, NVC)                                                                                                        \
   do {                                                                                                                      \
     constexpr size_t lds = (size_t)2 * Tile<NKS>::SIZE * sizeof(bf16_t);                                                    \

@@ -334,8 +334,8 @@ int launch_stream(const void* A, const void* W, void* C, int M, int N, int K, lo
 
 // bf16 operands of more than 8 rows whose rows come in whole 16-byte pieces, on v_mfma_f32_16x16x32_bf16 with fp32 sums: per-head maps as
 // batch and products with fp32 results (the GEMMs of gemm_bf16.hip write bf16).  A wave owns 32 rows of A x 64 rows of W, a workgroup
-// 64 x 128; operands come straight from global memory in the operand layout (the W rows of a tile are shared through the caches), a lane
-// ends with 4 neighbouring outputs of one row.
+// 64 x 128; operands come straight from global memory in the operand layout (the W rows of a tile are shared through the caches), the W rows
+// dealt out so that a lane ends with 16 neighbouring outputs of one row.
 template <typename TC>
 __global__ __launch_bounds__(256) void linear_any_mfma_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, TC* __restrict__ C, int M,
                                                               int N, int K, long lda, long ldw, long ldc, long sA, long sW, long sC,
@@ -351,7 +351,7 @@ __global__ __launch_bounds__(256) void linear_any_mfma_kernel(const bf16_t* __re
 #pragma unroll
   for (int i = 0; i < 2; ++i) ar[i] = A + (long)min(m0 + 16 * i + r16, M - 1) * lda + 8 * g;
 #pragma unroll
-  for (int j = 0; j < 4; ++j) wr[j] = W + (long)min(n0 + 16 * j + r16, N - 1) * ldw + 8 * g;
+  for (int j = 0; j < 4; ++j) wr[j] = W + (long)min(n0 + (r16 >> 2) * 16 + 4 * j + (r16 & 3), N - 1) * ldw + 8 * g;   // (operand row 4 g + r of product j)
   f32x4_t acc[2][4];
 #pragma unroll
   for (int i = 0; i < 2; ++i)
@@ -394,7 +394,7 @@ __global__ __launch_bounds__(256) void linear_any_mfma_kernel(const bf16_t* __re
     if (m >= M) continue;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      const int n = n0 + 16 * j + 4 * g;
+      const int n = n0 + 16 * g + 4 * j;                 // (a lane's four products: 16 neighbouring columns)
       TC* c = C + (long)m * ldc + n;
       if (n + 4 <= N && !accumulate && (((uintptr_t)c) & (4 * sizeof(TC) - 1)) == 0) {
         if constexpr (sizeof(TC) == 4) *reinterpret_cast<float4*>(c) = make_float4(acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]);

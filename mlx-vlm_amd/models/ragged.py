@@ -112,10 +112,10 @@ class DecodeRows:
 class RaggedLanguageModel:
     NAME = "model"
     MAX_DECODE_ROWS = 64
-    # steps of up to this many rows run their big projections on the weight-streaming kernels (with the expert skip); wider
-    # steps take the MFMA GEMM (measured: 1 / 2 / 4 / 8 rows 0.86 / 1.05 / 1.25 / 1.34 ms per step at width 1536 with 2, against
-    # 1.39 / 2.11 ms at 4 / 8 rows with 8).  Environment override for measurements.
-    STREAM_ROWS = int(os.environ.get("VLM_STREAM_ROWS") or os.environ.get("VLM_GARESUN_STREAM_ROWS") or "2")
+    # steps of up to this many rows run their big projections on the weight-streaming kernel (with the expert skip); wider steps take
+    # the MFMA GEMM (measured on six Rorovik layers of width 1536: 2 / 4 / 8 rows 0.62 / 0.88 / 1.35 ms per step streaming, 0.93 / 0.96 /
+    # 1.00 ms on the GEMM).  Environment override for measurements.
+    STREAM_ROWS = int(os.environ.get("VLM_STREAM_ROWS") or os.environ.get("VLM_GARESUN_STREAM_ROWS") or "4")
     STATEFUL = True                # recurrent layers: a step that ran cannot be taken back by moving the cache offset
     supports_logits_to_keep = True
 
