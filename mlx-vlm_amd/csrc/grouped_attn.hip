@@ -167,10 +167,10 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
     h0 = kh * R + o;
     ncol = min(heads_per_block, R - o);
   } else {
-    const int b = gridDim.x - 1 - blockIdx.x;            // (the blocks of a prompt's end have the most keys: they start first)
+    const int b = gridDim.y - 1 - blockIdx.y;            // (the blocks of a prompt's end have the most keys: they start first)
     t0 = p.qb_start[b];
     ncol = p.qb_count[b];
-    h0 = blockIdx.y * CG;
+    h0 = blockIdx.x * CG;
     kh = h0 / R;
   }
   const int* bt = p.block_table + (long)p.tok_seq[t0] * p.max_pages;
@@ -433,17 +433,17 @@ extern "C" int vlm_qkv_rownorm_rows(const vlm_qkv_rownorm_args* a, int rows, int
 
 extern "C" int vlm_grouped_attn_blocks(const vlm_grouped_attn_args* a, int nblocks, int dtype, void* stream) {
   if (bad(a) || !a->qb_start || !a->qb_count || nblocks < 0) return VLM_ERR_ARG;
-  if (a->H > 65535) return VLM_ERR_SHAPE;
+  if (a->H > 65535 || nblocks > 65535) return VLM_ERR_SHAPE;
   if (nblocks == 0) return VLM_OK;
   hipStream_t st = (hipStream_t)stream;
   if ((a->H / a->KH) % 2 == 0) {                         // two heads share the loaded keys and values
     const int NB = (a->Dv + 15) / 16 <= 8 ? 8 : 16;
     if (lds_bytes(*a, NB, 2, 4, dtype != 0) <= 64 * 1024) {
-      const dim3 grid(nblocks, a->H / 2);
+      const dim3 grid(a->H / 2, nblocks);
       return dtype ? launch<float, 2, 4>(*a, grid, 0, 16, st) : launch<bf16_t, 2, 4>(*a, grid, 0, 16, st);
     }
   }
-  const dim3 grid(nblocks, a->H);
+  const dim3 grid(a->H, nblocks);
   return dtype ? launch<float, 1, 4>(*a, grid, 0, 16, st) : launch<bf16_t, 1, 4>(*a, grid, 0, 16, st);
 }
 

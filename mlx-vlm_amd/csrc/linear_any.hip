@@ -358,7 +358,7 @@ __global__ __launch_bounds__(256) void linear_any_mfma_kernel(const bf16_t* __re
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   const int K32 = K & ~31;
-#pragma unroll 2
+#pragma unroll 4
   for (int k = 0; k < K32; k += 32) {
     bf8 a[2], w[4];
 #pragma unroll
