@@ -158,7 +158,7 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r16 = lane & 15, g = lane >> 4;
   const int R = p.H / p.KH;
   // the workgroup's columns: column c of group m is (token t0 + c, head h0 + m), decoding (token t0, head h0 + c)
-  int t0, ncol, h0, kh;
+  int t0, ncol, h0, kh, nm = CG;                         // (nm: groups that exist)
   if (decode) {
     const int hb = (R + heads_per_block - 1) / heads_per_block;
     t0 = blockIdx.x;
@@ -170,8 +170,10 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
     const int b = gridDim.y - 1 - blockIdx.y;            // (the blocks of a prompt's end have the most keys: they start first)
     t0 = p.qb_start[b];
     ncol = p.qb_count[b];
-    h0 = blockIdx.x * CG;
-    kh = h0 / R;
+    const int hp = (R + CG - 1) / CG, o = (blockIdx.x % hp) * CG;
+    kh = blockIdx.x / hp;
+    h0 = kh * R + o;
+    nm = min(CG, R - o);
   }
   const int* bt = p.block_table + (long)p.tok_seq[t0] * p.max_pages;
   const int pos0 = p.tok_pos[t0], last = decode ? pos0 : pos0 + ncol - 1;
@@ -192,7 +194,7 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
   for (int i = tid; i < CG * QC * dq; i += NW * 64) {
     const int d = i % dq, c = (i / dq) % QC, m = i / (dq * QC);
     float v = 0.f;
-    if (c < ncol && d < D) {
+    if (c < ncol && d < D && m < nm) {
       const long tok = decode ? t0 : t0 + c;
       const int h = decode ? h0 + c : h0 + m;
       v = p.q[(tok * p.H + h) * D + d] * sc;
@@ -209,7 +211,7 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
   const int mypos = r16 < ncol ? (decode ? pos0 : pos0 + r16) : -1;       // (a column that does not exist sees nothing)
   float slope[CG];                                       // of this lane's column, times log2(e)
 #pragma unroll
-  for (int m = 0; m < CG; ++m) slope[m] = p.slope ? p.slope[decode ? h0 + min(r16, ncol - 1) : h0 + m] * LOG2E : 0.f;
+  for (int m = 0; m < CG; ++m) slope[m] = p.slope ? p.slope[decode ? h0 + min(r16, ncol - 1) : h0 + min(m, nm - 1)] * LOG2E : 0.f;
   f32x4_t acc[CG][NB];
 #pragma unroll
   for (int m = 0; m < CG; ++m)
@@ -324,7 +326,7 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
     const float ms = M == -INFINITY ? 0.f : M;
     float l = 0.f;
     for (int w = 0; w < NW; ++w) l = fmaf(ml[((w * CG + m) * QC + r16) * 2 + 1], __builtin_amdgcn_exp2f(ml[((w * CG + m) * QC + r16) * 2] - ms), l);
-    const int h = decode ? h0 + min(r16, ncol - 1) : h0 + m;
+    const int h = decode ? h0 + min(r16, ncol - 1) : h0 + min(m, nm - 1);
     if (split) {
       if (wave == 0 && g == 0 && r16 < ncol) {           // (split only when decoding: CG = 1)
         float* q = p.part + (((long)blockIdx.z * p.H + h) * gridDim.x + t0) * (Dv + 2);
@@ -354,7 +356,7 @@ __global__ __launch_bounds__(NW * 64) void grouped_attn_kernel(vlm_grouped_attn_
     }
     __syncthreads();
   }
-  for (int i = tid; i < CG * ncol * Dv; i += NW * 64) {
+  for (int i = tid; i < nm * ncol * Dv; i += NW * 64) {
     const int d = i % Dv, c = (i / Dv) % ncol, m = i / (Dv * ncol);
     const long tok = decode ? t0 : t0 + c;
     const int h = decode ? h0 + c : h0 + m;
@@ -436,10 +438,11 @@ extern "C" int vlm_grouped_attn_blocks(const vlm_grouped_attn_args* a, int nbloc
   if (a->H > 65535 || nblocks > 65535) return VLM_ERR_SHAPE;
   if (nblocks == 0) return VLM_OK;
   hipStream_t st = (hipStream_t)stream;
-  if ((a->H / a->KH) % 2 == 0) {                         // two heads share the loaded keys and values
+  const int R = a->H / a->KH;
+  if (R >= 2) {                                          // two heads share the loaded keys and values (an odd one runs alone)
     const int NB = (a->Dv + 15) / 16 <= 8 ? 8 : 16;
     if (lds_bytes(*a, NB, 2, 4, dtype != 0) <= 64 * 1024) {
-      const dim3 grid(a->H / 2, nblocks);
+      const dim3 grid(a->KH * ((R + 1) / 2), nblocks);
       return dtype ? launch<float, 2, 4>(*a, grid, 0, 16, st) : launch<bf16_t, 2, 4>(*a, grid, 0, 16, st);
     }
   }

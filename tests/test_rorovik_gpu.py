@@ -813,24 +813,27 @@ def test_trace_replay_program_writes_the_asked_logits(tmp_path, dtype):
         assert got.shape == w.shape and H.rel_rms(got, w) < 2.5 * TOL[dtype], n
 
 
-@pytest.mark.parametrize("rows", [1, 3])
+@pytest.mark.parametrize("rows", [1, 3, 12, 64])
 def test_captured_decode_steps_equal_eager_ones(tmp_path, rows):
     """a captured decode step is replayed many times, with eager work (another request's prompt, a release, synchronisations)
-    between the replays; every replay's logits and token must equal the eager step's"""
+    between the replays; every replay's logits and token must equal the eager step's.  12 and 64 rows: the prompt forms of the attentions
+    and the experts pair by pair inside a captured step."""
     from mlx_vlm_amd.sample_utils import make_sampler
 
-    cfg = H.mixed_config()
+    pairs = [H.attention(window=70, mlp=H.moe(experts=6, identity=2, top=3, ff=64)), H.latent(mlp=H.moe(experts=4, identity=0, top=2, ff=64)), H.attention(heads=2)]
+    cfg = H.mixed_config() if rows < 64 else H.config(pairs, width=64)
     W = H.weights(cfg, seed=71)
-    lm = _load(tmp_path, cfg, W, "bfloat16", tokens=2048, seqs=6).language_model
+    lm = _load(tmp_path, cfg, W, "bfloat16", tokens=16384, seqs=rows + 3).language_model
     sargs = make_sampler().engine_args()
-    prompts = [_ids(n, cfg["vocab"], 80 + n) for n in (40, 7, 66)[:rows]]
+    prompts = [_ids(n, cfg["vocab"], 80 + n) for n in ([40, 7, 66] * 22)[:rows]]
+    steps = 70 if rows < 64 else 20
 
     def run(use_graph):
         caches = lm.make_cache_batch(rows)
         lg = lm.prefill(torch.cat([torch.as_tensor(p) for p in prompts]).cuda().reshape(-1, 1), None, caches, [len(p) for p in prompts])
         st = lm.decode_begin(caches, lg.argmax(-1), np.zeros((rows, 1)), max_new_tokens=80)
         out = []
-        for i in range(70):                                          # crosses a page border and the windows in every row
+        for i in range(steps):                                       # crosses a page border and the windows in every row
             lm.decode_run(st, 1, sargs, use_graph=use_graph)
             out.append((st.tok.cpu().clone(), st.logits.float().cpu().clone()))
             if i % 9 == 4:                                           # eager work between replays
