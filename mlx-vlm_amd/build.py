@@ -3,8 +3,7 @@
     python mlx-vlm_amd/build.py [--force]
 
 Sources: mlx-vlm_amd/csrc/*.hip  ->  mlx-vlm_amd/lib/libvlm_hip.so
-hipcc cross-compiles for gfx950 without a GPU; the .so travels to the GPU box
-with the repo snapshot (it is git-ignored, not gpurun-ignored).
+hipcc cross-compiles for gfx950 without a GPU; the .so is git-ignored.
 """
 from __future__ import annotations
 

@@ -8,7 +8,7 @@ from dataclasses import dataclass, field
 from typing import Any, Dict, List, Optional
 
 MIXERS = ("attention", "latent_attention")
-MAX_VDIM, MAX_RANK, MAX_EXPERTS = 256, 1024, 256          # what the kernels take
+MAX_VDIM, MAX_DIM, MAX_RANK, MAX_EXPERTS = 256, 768, 1024, 256          # what the kernels take
 
 
 def _need(d: Dict[str, Any], keys, what: str):
@@ -33,8 +33,8 @@ class LayerConfig:
             m.setdefault("vdim", m["dim"])
             if min(int(m["kv_heads"]), int(m["dim"]), int(m["vdim"])) < 1 or int(m["heads"]) % int(m["kv_heads"]):
                 raise ValueError("attention mixer: heads must be a multiple of kv_heads, sizes at least 1")
-            if int(m["vdim"]) > MAX_VDIM or int(m["dim"]) > 4 * MAX_VDIM:
-                raise ValueError(f"attention mixer: vdim up to {MAX_VDIM}, dim up to {4 * MAX_VDIM}")
+            if int(m["vdim"]) > MAX_VDIM or int(m["dim"]) > MAX_DIM:
+                raise ValueError(f"attention mixer: vdim up to {MAX_VDIM}, dim up to {MAX_DIM}")
             qt = m.get("q_temp")
             if qt is not None:
                 _need(qt, ("coef", "every"), "attention mixer, q_temp")

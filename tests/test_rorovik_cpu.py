@@ -31,7 +31,7 @@ def test_config_reads_every_size_and_refuses_what_the_design_does_not_have():
     ModelConfig.from_dict(H.config([dict(H.latent(mlp=None), mlp=None)]))
     no_scale = H.attention()
     del no_scale["mixer"]["scale"]
-    for layers in ([dict(H.latent(), type="lightning")], [H.attention(heads=5, kv_heads=2)], [H.attention(window=-3)], [H.attention(every=-1)], [H.attention(vdim=300)],
+    for layers in ([dict(H.latent(), type="lightning")], [H.attention(heads=5, kv_heads=2)], [H.attention(window=-3)], [H.attention(every=-1)], [H.attention(vdim=300)], [H.attention(dim=800)],
                    [no_scale], [H.latent(rot_dim=5)], [dict(H.latent(), mixer=dict(H.latent()["mixer"], rot=dict(base=5.0, dims=4)))],
                    [dict(H.latent(), mixer={k: v for k, v in H.latent()["mixer"].items() if k != "rot"})], [H.latent(scaling=dict(factor=2.0))],
                    [H.latent(kv_rank=1100)], [H.latent(q_rank=0)], [H.latent(mlp=H.moe(experts=2, identity=1, top=4))], [H.latent(mlp=H.moe(experts=0, identity=3))],

@@ -273,7 +273,7 @@ def _pool_case(g, deep=1890):
 
 
 @pytest.mark.parametrize("D,Dv,Hh,G", [(12, 20, 6, 2), (16, 16, 2, 2), (6, 33, 3, 1), (40, 72, 20, 1), (64, 128, 6, 2), (128, 128, 12, 2), (1, 1, 1, 1),
-                                       (18, 256, 2, 1), (256, 256, 1, 1), (72, 136, 4, 2)])
+                                       (18, 256, 2, 1), (256, 256, 1, 1), (72, 136, 4, 2), (768, 24, 7, 1)])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_grouped_attention_bias_window_sink_and_gate_against_a_dense_softmax(dtype, D, Dv, Hh, G):
     from mlx_vlm_amd import ops
