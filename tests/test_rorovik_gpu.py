@@ -111,7 +111,7 @@ def test_sandwich_step_norms_the_result_adds_it_and_forms_the_next_input(T, D):
     assert (xd.cpu().double() - new).abs().max() < 3e-5 and (h.cpu().double() - O.norm(new, d(w), 1e-3)).abs().max() < 4 * tol
 
 
-@pytest.mark.parametrize("D,E,identity,top", [(48, 6, 1, 2), (56, 3, 2, 3), (57, 14, 0, 4), (1536, 14, 2, 2), (64, 1, 1, 1), (64, 40, 3, 7), (128, 200, 56, 9),
+@pytest.mark.parametrize("D,E,identity,top", [(48, 6, 1, 2), (56, 3, 2, 3), (57, 14, 0, 4), (1536, 13, 3, 2), (64, 1, 1, 1), (64, 40, 3, 7), (128, 200, 56, 9),
                                               (64, 90, 0, 90), (3584, 64, 8, 6)])
 @pytest.mark.parametrize("T", [torch.float32, torch.bfloat16])
 def test_router_scores_correction_and_identity_experts(T, D, E, identity, top):
@@ -322,7 +322,7 @@ def test_grouped_attention_bias_window_sink_and_gate_against_a_dense_softmax(dty
             assert (a.cpu().double().view(42, Hh, Dv) - want).abs().max() < tol, (window, nsplit)
 
 
-@pytest.mark.parametrize("R,Dr,Hh", [(40, 8, 3), (21, 4, 2), (512, 64, 12), (128, 16, 8), (264, 2, 2), (96, 32, 20), (24, 0, 1), (520, 8, 2), (16, 16, 33)])
+@pytest.mark.parametrize("R,Dr,Hh", [(40, 8, 3), (21, 4, 2), (512, 64, 12), (136, 24, 10), (264, 2, 2), (96, 32, 20), (24, 0, 1), (520, 8, 2), (16, 16, 33)])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_latent_attention_with_sinks_every_form_against_a_dense_softmax(dtype, R, Dr, Hh):
     from mlx_vlm_amd import ops
